@@ -20,6 +20,7 @@ from .taluvik import ARCHITECTURE as TALUVIK, TaluvikConfig, taluvik_model_spec
 from .vobolorn import ARCHITECTURE as VOBOLORN, VobolornConfig, vobolorn_model_spec
 from .kepevik import ARCHITECTURE as KEPEVIK, KepevikConfig, kepevik_model_spec, kepevik_sizes_from_tensors
 from .nosuzen import ARCHITECTURE as NOSUZEN, NosuzenConfig, nosuzen_model_spec, nosuzen_sizes_from_tensors
+from .rifizen import ARCHITECTURE as RIFIZEN, RifizenConfig, rifizen_model_spec
 
 
 @dataclass(frozen=True)
@@ -248,5 +249,28 @@ register_architecture(
         stop_token_ids=_nosuzen_stop_ids,
         config_type=NosuzenConfig,
         sizes_from_tensors=nosuzen_sizes_from_tensors,
+    )
+)
+
+
+def _rifizen_rules(cfg: RifizenConfig):
+    from ..weights.names import rifizen_name_rules
+
+    return rifizen_name_rules(cfg)
+
+
+def _rifizen_stop_ids(cfg: RifizenConfig):
+    eos = cfg.eos_token_id
+    return [] if eos is None else (list(eos) if isinstance(eos, (list, tuple)) else [eos])
+
+
+register_architecture(
+    ArchSpec(
+        name=RIFIZEN,
+        config_from_dict=RifizenConfig.from_dict,
+        model_spec=rifizen_model_spec,
+        weight_rules=_rifizen_rules,
+        stop_token_ids=_rifizen_stop_ids,
+        config_type=RifizenConfig,
     )
 )

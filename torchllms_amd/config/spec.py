@@ -57,10 +57,14 @@ class LayerRun:
     ``layer`` indexes ``ModelSpec.layers`` (a layer may appear in several runs and then
     shares its weights between them).  Every run owns a cache entry of its own unless
     ``cache_from`` names an earlier run: then this run reads that run's cache and writes none.
+    ``step_vector`` t: row t of the model's step vectors (``ModelSpec.step_vectors``) is added to the
+    residual stream right before this run (layers that run several times in a row may so be told
+    which pass it is).
     """
 
     layer: int
     cache_from: Optional[int] = None
+    step_vector: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -74,12 +78,16 @@ class ModelSpec:
     order: List[LayerRun]
     final_norm: PartSpec
     head: PartSpec
+    #: how many vectors of the model's width (the tensor ``loop.step``) runs may name with ``LayerRun.step_vector``
+    step_vectors: int = 0
 
     def validate(self) -> None:
         n = len(self.layers)
         for i, run in enumerate(self.order):
             if not 0 <= run.layer < n:
                 raise ValueError(f"order[{i}] names layer {run.layer}, but the model has {n} layers")
+            if run.step_vector is not None and not 0 <= run.step_vector < self.step_vectors:
+                raise ValueError(f"order[{i}] names step vector {run.step_vector}, but the model has {self.step_vectors}")
             if run.cache_from is not None:
                 if not 0 <= run.cache_from < i:
                     raise ValueError(

@@ -87,6 +87,7 @@ struct DecodeArgs {
   float cap_log2e;    // > 0: scores are capped, cap * tanh(score / cap); this is cap * log2(e) ...
   float two_scale_over_cap_log2e;  // ... and this 2 * scale / cap * log2(e): tanh(x) = 1 - 2 / (exp2(2 x log2(e)) + 1)
   const float* sinks;  // per query head, or null: exp(sink) joins the softmax's denominator
+  const float* slopes; // per query head, or null: what a capped score loses for every position between key and query
   int split_size;     // keys per split, a multiple of 64
   int n_splits;
   float* ws_o;   // [token][q head][split][DH]
@@ -179,6 +180,8 @@ __global__ void __launch_bounds__(kWaves* kWave, TL_DECODE_MIN_WAVES) attn_decod
       if (n16 >= R) qreg[u].u = u32x4_t{0, 0, 0, 0};
     }
   }
+
+  const float slope_log2e = a.slopes ? a.slopes[kvh * R + (n16 < R ? n16 : 0)] * 1.4426950408889634f : 0.f;
 
   float m_run = -INFINITY;  // running maximum of head n16 (same in the four g4 lanes)
   float l_part = 0.f;       // sum of this lane's own probabilities
@@ -274,6 +277,7 @@ __global__ void __launch_bounds__(kWaves* kWave, TL_DECODE_MIN_WAVES) attn_decod
       float sc = c[i] * a.scale_log2e;
       if (a.cap_log2e > 0.f)  // (the same in every lane)
         sc = a.cap_log2e * (1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(c[i] * a.two_scale_over_cap_log2e) + 1.0f));
+      sc = fmaf(-slope_log2e, (float)(p - (count < keep_al ? count : key)), sc);
       s[i] = valid ? sc : -INFINITY;
       tmax = fmaxf(tmax, s[i]);
     }
@@ -420,7 +424,7 @@ TL_EXPORT int tl_attn_decode_head_dim() { return DH; }
 
 // q: element (t, h, d) at q + t*q_stride + h*DH + d; out likewise.  Pages [page][Hkv][page_size][DH].
 // softcap > 0 caps the scores, chunk > 0 confines a query to its chunk, sinks (one float per query head, or
-// null) join the denominators.  Every token is one query at positions[t] of request row token_seq[t].  split_size: keys per
+// null) join the denominators, slopes (likewise) are taken off the capped scores for every position of distance.  Every token is one query at positions[t] of request row token_seq[t].  split_size: keys per
 // split (a multiple of 64); n_splits >= ceil(longest visible range / split_size), counted from the
 // 16-aligned first visible key, plus the kept first keys rounded up to 16.  keep_first, n_v_heads (0: n_kv_heads),
 // v_pitch / v_offset and out_pitch / out_offset (0: DH): see DecodeArgs.  ws_o / ws_ml: workspaces (unused when n_splits == 1).
@@ -430,7 +434,7 @@ TL_EXPORT int tl_attn_decode(const void* q, int q_stride, void* out, int out_str
                              int n_kv_heads, int head_dim, int page_size, int window, float scale,
                              int split_size, int n_splits, float* ws_o, float* ws_ml, float softcap, int chunk,
                              const float* sinks, int keep_first, int n_v_heads, int v_pitch, int v_offset, int out_pitch,
-                             int out_offset, hipStream_t stream) {
+                             int out_offset, const float* slopes, hipStream_t stream) {
   if (head_dim != DH) return variant_fail(TL_ERR_ARG, "attn_decode: built for head_dim %d, called with %d", DH, head_dim);
   if (n_tokens < 0 || n_q_heads <= 0 || n_kv_heads <= 0 || page_size <= 0 || bt_stride <= 0 || window < 0 || chunk < 0 || softcap < 0)
     return variant_fail(TL_ERR_ARG, "attn_decode: bad sizes");
@@ -458,7 +462,7 @@ TL_EXPORT int tl_attn_decode(const void* q, int q_stride, void* out, int out_str
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == page_size) a.page_shift = sh;
   a.scale_log2e = scale * 1.4426950408889634f;
-  a.chunk = chunk; a.sinks = sinks;
+  a.chunk = chunk; a.sinks = sinks; a.slopes = slopes;
   a.keep_first = keep_first; a.n_v_heads = n_v_heads; a.v_pitch = v_pitch; a.v_offset = v_offset;
   a.out_pitch = out_pitch; a.out_offset = out_offset;
   a.cap_log2e = softcap > 0 ? softcap * 1.4426950408889634f : 0.f;

@@ -9,7 +9,8 @@
 // per query head (one more term exp(sink) in the softmax's denominator, without a value), first keys that stay
 // visible behind a window (keep_first: a query also sees the positions below it that lie before its window), and
 // values with fewer heads than the keys (key head g reads value head g mod n_v_heads: several score maps over
-// the same values).
+// the same values), and a bias by distance (slopes: a number per query head that is taken off the capped score for
+// every position between key and query).
 #include <limits.h>
 
 #include "common.h"
@@ -59,6 +60,8 @@ struct Query {
   int lo, p;                // the keys it sees: positions lo .. p
   int keep;                 // and positions 0 .. keep - 1 before them (kept first keys; keep <= lo)
   float scale, softcap;
+  int pos;                  // the query's position, and what a position of distance costs its head
+  float slope;
 };
 
 // The first position a query at position p sees: behind a window of `window` keys (0: none) and inside
@@ -121,7 +124,7 @@ __device__ __forceinline__ void block_partial(const Query<T>& a, int j0, int lan
     } else {
       for (int d = 0; d < a.head_dim; ++d) dot = fmaf(a.qs[d], to_f32(kr[d]), dot);
     }
-    s = capped(dot * a.scale, a.softcap);
+    s = capped(dot * a.scale, a.softcap) - a.slope * (float)(a.pos - j);
   }
   m_b = wave_max(s);
   const float pj = valid ? expf(s - m_b) : 0.f;
@@ -179,7 +182,7 @@ __device__ __forceinline__ Query<T> make_query(const float* qs, const T* k_pages
                                                const int32_t* block_table, int bt_stride, int t, int h, int n_q_heads,
                                                int n_kv_heads, int head_dim, int page_size, int window, float scale,
                                                float softcap, int chunk, int v_dim, int v_pitch, int keep_first,
-                                               int n_v_heads) {
+                                               int n_v_heads, const float* slopes) {
   Query<T> a;
   a.qs = qs; a.k_pages = k_pages; a.v_pages = v_pages;
   a.bt = block_table + (size_t)token_seq[t] * bt_stride;
@@ -190,6 +193,8 @@ __device__ __forceinline__ Query<T> make_query(const float* qs, const T* k_pages
   a.keep = min(keep_first, a.lo);
   a.n_v_heads = n_v_heads; a.gv = a.g % n_v_heads;
   a.scale = scale; a.softcap = softcap;
+  a.pos = a.p;
+  a.slope = slopes ? slopes[h] : 0.f;
   return a;
 }
 
@@ -223,7 +228,8 @@ attention_generic_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ 
                          const int32_t* __restrict__ token_seq, const int32_t* __restrict__ positions,
                          const int32_t* __restrict__ block_table, int bt_stride, int n_q_heads,
                          int n_kv_heads, int head_dim, int page_size, int window, float scale, float softcap,
-                         int chunk, const float* __restrict__ sinks, int v_dim, int v_pitch, int keep_first, int n_v_heads) {
+                         int chunk, const float* __restrict__ sinks, int v_dim, int v_pitch, int keep_first, int n_v_heads,
+                         const float* __restrict__ slopes) {
   __shared__ float q_lds[kWavesPerBlock][kMaxKeyDim];
   const int t = blockIdx.x;
   const int wave = threadIdx.x / kWave;
@@ -235,7 +241,8 @@ attention_generic_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ 
   for (int d = lane; d < head_dim; d += kWave) q_lds[wave][d] = to_f32(qv[d]);
   __syncthreads();
   const Query<T> a = make_query<T>(q_lds[wave], k_pages, v_pages, token_seq, positions, block_table, bt_stride, t, h,
-                                   n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, v_dim, v_pitch, keep_first, n_v_heads);
+                                   n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, v_dim, v_pitch, keep_first, n_v_heads,
+                                   slopes);
   float acc[kChanPerLane];
 #pragma unroll
   for (int c = 0; c < kChanPerLane; ++c) acc[c] = 0.f;
@@ -265,7 +272,7 @@ constexpr int kTilePad = 4;  // floats between LDS rows beyond head_dim: rows st
 template <bool VEC, int CH>
 __device__ __forceinline__ void block_partial_lds(const float* qs, const float* k_t, const float* v_t, int pitch,
                                                   int pitch_v, int head_dim, int v_dim, int lo, int p, float scale,
-                                                  float softcap, int j0, int lane,
+                                                  float softcap, float slope, int pos, int j0, int lane,
                                                   float& m_b, float& l_b, float (&o_b)[kChanPerLane]) {
 #pragma clang fp contract(off)
   const int j = j0 + lane;
@@ -284,7 +291,7 @@ __device__ __forceinline__ void block_partial_lds(const float* qs, const float* 
     } else {
       for (int d = 0; d < head_dim; ++d) dot = fmaf(qs[d], kr[d], dot);
     }
-    s = capped(dot * scale, softcap);
+    s = capped(dot * scale, softcap) - slope * (float)(pos - j);
   }
   m_b = wave_max(s);
   const float pj = valid ? expf(s - m_b) : 0.f;
@@ -330,7 +337,7 @@ attention_tile_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ out
                       const int32_t* __restrict__ block_table, int bt_stride, int n_tokens, int n_q_heads,
                       int n_kv_heads, int head_dim, int page_size, int window, float scale, int heads_per_block,
                       float softcap, int chunk, const float* __restrict__ sinks, int v_dim, int v_pitch, int keep_first,
-                      int n_v_heads) {
+                      int n_v_heads, const float* __restrict__ slopes) {
   extern __shared__ __attribute__((aligned(16))) float tile_lds[];
   const int pitch = head_dim + kTilePad, pitch_v = v_dim + kTilePad;
   float* q_lds = tile_lds;                          // [kTileWaves][head_dim]
@@ -350,7 +357,7 @@ attention_tile_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ out
   for (int d = lane; d < head_dim; d += kWave) q_lds[wave * head_dim + d] = to_f32(qv[d]);
   const Query<T> a = make_query<T>(q_lds + wave * head_dim, k_pages, v_pages, token_seq, positions, block_table,
                                    bt_stride, t, h, n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap,
-                                   chunk, v_dim, v_pitch, keep_first, n_v_heads);
+                                   chunk, v_dim, v_pitch, keep_first, n_v_heads, slopes);
   // what the whole block sees: the same for every thread, from the tokens' own entries
   const int last = min(t0 + QT, n_tokens) - 1;
   const int seq0 = token_seq[t0];
@@ -411,7 +418,7 @@ attention_tile_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ out
       __syncthreads();
       if (p_w >= lo_w && j0 >= lo_w - lo_w % kWave && j0 <= p_w) {  // (uniform per wave)
         float m_b, l_b, o_b[kChanPerLane];
-        block_partial_lds<VEC, CH>(a.qs, k_t, v_t, pitch, pitch_v, head_dim, v_dim, lo_w, p_w, scale, softcap, j0, lane,
+        block_partial_lds<VEC, CH>(a.qs, k_t, v_t, pitch, pitch_v, head_dim, v_dim, lo_w, p_w, scale, softcap, a.slope, a.pos, j0, lane,
                                    m_b, l_b, o_b);
         merge_block(m, l, acc, m_b, l_b, o_b);
       }
@@ -443,7 +450,7 @@ attention_blocks_kernel(const T* __restrict__ q, int q_stride, const T* __restri
                         const int32_t* __restrict__ positions, const int32_t* __restrict__ block_table, int bt_stride,
                         int n_q_heads, int n_kv_heads, int head_dim, int page_size, int window, float scale,
                         float* __restrict__ partials, int max_blocks, float softcap, int chunk, int v_dim, int v_pitch,
-                        int keep_first, int n_v_heads) {
+                        int keep_first, int n_v_heads, const float* __restrict__ slopes) {
   __shared__ float q_lds[kWavesPerBlock][kMaxKeyDim];
   const int t = blockIdx.x;
   const int r = blockIdx.z;
@@ -456,7 +463,8 @@ attention_blocks_kernel(const T* __restrict__ q, int q_stride, const T* __restri
   for (int d = lane; d < head_dim; d += kWave) q_lds[wave][d] = to_f32(qv[d]);
   __syncthreads();
   const Query<T> a = make_query<T>(q_lds[wave], k_pages, v_pages, token_seq, positions, block_table, bt_stride, t, h,
-                                   n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, v_dim, v_pitch, keep_first, n_v_heads);
+                                   n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, v_dim, v_pitch, keep_first, n_v_heads,
+                                   slopes);
   // the blocks of the kept first keys come first, then those of positions lo .. p
   const int kept_blocks = (a.keep + kWave - 1) / kWave;
   Query<T> b = a;
@@ -533,14 +541,15 @@ attention_join_kernel(T* __restrict__ out, int out_stride, const int32_t* __rest
 
 // q: element (t, h, d) at q + t*q_stride + h*head_dim + d.  out likewise with out_stride.
 // pages: [page][n_kv_heads][page_size][head_dim].  token_seq[t]: row of block_table;
-// positions[t]: absolute position; the token sees positions max(0, p-window+1)..p (window 0: all).
+// positions[t]: absolute position; the token sees positions max(0, p-window+1)..p (window 0: all).  slopes: one float
+// per query head (or null) that a capped score loses for every position between its key and the query.
 TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int out_stride,
                                    const void* k_pages, const void* v_pages, const int32_t* token_seq,
                                    const int32_t* positions, const int32_t* block_table, int bt_stride,
                                    int n_tokens, int n_q_heads, int n_kv_heads, int head_dim,
                                    int page_size, int window, float scale, float softcap, int chunk,
                                    const float* sinks, int v_dim, int v_pitch, int dtype, int keep_first, int n_v_heads,
-                                   hipStream_t stream) {
+                                   const float* slopes, hipStream_t stream) {
   TL_REQUIRE(n_tokens >= 0 && n_q_heads > 0 && n_kv_heads > 0 && page_size > 0 && bt_stride > 0,
              "attention: bad sizes");
   TL_REQUIRE(n_q_heads % n_kv_heads == 0, "attention: %d query heads are not a multiple of %d kv heads",
@@ -577,7 +586,7 @@ TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int o
     attention_tile_kernel<T, VEC, CH><<<tgrid, kTileWaves * kWave, lds, stream>>>(                               \
         (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pages, (const T*)v_pages, token_seq, positions,  \
         block_table, bt_stride, n_tokens, n_q_heads, n_kv_heads, head_dim, page_size, window, scale, hb, softcap, \
-        chunk, sinks, v_dim, v_pitch, keep_first, n_v_heads);                                                    \
+        chunk, sinks, v_dim, v_pitch, keep_first, n_v_heads, slopes);                                            \
   } while (0)
 #define TL_TILE_LAUNCH(T, VEC)                                                                                   \
   do {                                                                                                           \
@@ -603,7 +612,7 @@ TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int o
   attention_generic_kernel<T, VEC><<<grid, kWavesPerBlock * kWave, 0, stream>>>(                            \
       (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pages, (const T*)v_pages, token_seq, positions, \
       block_table, bt_stride, n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, sinks, v_dim, v_pitch, \
-      keep_first, n_v_heads)
+      keep_first, n_v_heads, slopes)
   if (dtype == TL_F32) {
     if (vec) TL_ATTN_LAUNCH(float, true);
     else TL_ATTN_LAUNCH(float, false);
@@ -627,7 +636,8 @@ TL_EXPORT int tl_attention_generic_split(const void* q, int q_stride, void* out,
                                          int n_tokens, int n_q_heads, int n_kv_heads, int head_dim,
                                          int page_size, int window, float scale, float softcap, int chunk,
                                          const float* sinks, int v_dim, int v_pitch, int dtype, int max_blocks,
-                                         float* partials, int keep_first, int n_v_heads, hipStream_t stream) {
+                                         float* partials, int keep_first, int n_v_heads, const float* slopes,
+                                         hipStream_t stream) {
   TL_REQUIRE(n_tokens >= 0 && n_q_heads > 0 && n_kv_heads > 0 && page_size > 0 && bt_stride > 0,
              "attention: bad sizes");
   TL_REQUIRE(n_q_heads % n_kv_heads == 0, "attention: %d query heads are not a multiple of %d kv heads",
@@ -654,7 +664,7 @@ TL_EXPORT int tl_attention_generic_split(const void* q, int q_stride, void* out,
     attention_blocks_kernel<T, VEC><<<grid, kWavesPerBlock * kWave, 0, stream>>>(                               \
         (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, token_seq, positions, block_table, bt_stride, \
         n_q_heads, n_kv_heads, head_dim, page_size, window, scale, partials, max_blocks, softcap, chunk, v_dim, v_pitch,  \
-        keep_first, n_v_heads);                                                                                 \
+        keep_first, n_v_heads, slopes);                                                                         \
     int rc = tl_check_launch("attention_blocks");                                                               \
     if (rc != TL_OK) return rc;                                                                                 \
     attention_join_kernel<T><<<grid_join, kWavesPerBlock * kWave, 0, stream>>>(                                 \

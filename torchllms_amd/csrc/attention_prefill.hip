@@ -109,6 +109,8 @@ struct PrefillArgs {
   float cap_over_scale;             // capped scores: s <- cap * tanh(s * scale / cap), taken on the raw product as
   float two_scale_over_cap_log2e;   // c <- (cap / scale) * (1 - 2 / (exp2(c * 2 scale / cap * log2(e)) + 1))
   const float* sinks;               // per query head, or null: exp(sink) joins the softmax's denominator
+  const float* slopes;              // per query head, or null: what a capped score loses for every position between key and query
+  float inv_scale;                  // 1 / softmax scale: the pipeline's scores are raw products
 };
 
 typedef unsigned int u32x2_t __attribute__((ext_vector_type(2)));
@@ -165,10 +167,11 @@ __device__ __forceinline__ u32x2_t lds_transposed(const bf16_t* src) {
 // they have at the end through LDS: a block's chain of tiles is half as long, which is what a launch
 // needs whose blocks all fit the GPU at once and whose time is therefore that of its longest block.
 // MODE 0: no lower bound and no cap; 1: a lower bound (a window, chunks, or both); 2: a lower bound and capped scores;
-// 3: a lower bound, and before it the first keep_first positions, which come as tiles of their own ahead of the others.
+// 3: a lower bound, and before it the first keep_first positions, which come as tiles of their own ahead of the others;
+// 4: a lower bound and a bias by distance; 5: a lower bound, capped scores and a bias by distance.
 template <int RP, int MODE, int GROUPS>
 __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) attn_prefill_kernel(PrefillArgs a) {
-  constexpr bool WINDOWED = MODE >= 1, CAPPED = MODE == 2, KEPT = MODE == 3;
+  constexpr bool WINDOWED = MODE >= 1, CAPPED = MODE == 2 || MODE == 5, KEPT = MODE == 3, BIASED = MODE >= 4;
   constexpr int QB = kCols / RP;  // queries per block
 
   const int tile = blockIdx.y;  // the host lists the tiles in the order that balances the launch
@@ -207,6 +210,7 @@ __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) 
   // this lane's columns: col -> (query, head)
   int col_pos[NC], col_lo[NC], col_tok[NC], col_head[NC];
   bool col_ok[NC];
+  float col_slope[NC];  // (BIASED) in units of the raw products
   Pack16 qreg[NC][KL];
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
@@ -219,6 +223,7 @@ __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) 
     // a column that stands for nothing sees every key with a zero query: finite, never stored
     col_pos[i] = col_ok[i] ? pos0 + ql : 0x3fffffff;
     col_lo[i] = col_ok[i] ? window_lo(pos0 + ql) : 0;
+    col_slope[i] = BIASED && col_ok[i] ? a.slopes[col_head[i]] * a.inv_scale : 0.f;
     const bf16_t* qrow = a.q + (size_t)col_tok[i] * a.q_stride + (size_t)col_head[i] * DH;
 #pragma unroll
     for (int u = 0; u < KL; ++u) {
@@ -472,6 +477,17 @@ __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) 
           for (int r = 0; r < 4; ++r)
             c[i][sub][r] = a.cap_over_scale * (1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(c[i][sub][r] * a.two_scale_over_cap_log2e) + 1.0f));
     }
+    if constexpr (BIASED) {
+      // c -= slope * (position - key), as what the lane's first key costs and a multiple of the slope for the others
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        const float first = col_slope[i] * (float)(col_pos[i] - base - 4 * g4);
+#pragma unroll
+        for (int sub = 0; sub < NS; ++sub)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) c[i][sub][r] = (c[i][sub][r] - first) + col_slope[i] * (float)(16 * sub + r);
+      }
+    }
     if (kept_of(step) || base + KT - 1 > pos0 + q0 || (WINDOWED && base < window_lo(pos0 + q_last))) mask(base, kept_of(step));
     softmax(pb, alpha, moved);
     output(v_tile(step - 1), pb_prev);
@@ -568,7 +584,7 @@ TL_EXPORT int tl_attn_prefill(const void* q, int q_stride, void* out, int out_st
                               const int32_t* tile_q0, int n_tiles, int n_q_heads, int n_kv_heads, int head_dim,
                               int page_size, int window, float scale, int key_groups, float softcap, int chunk,
                               const float* sinks, int keep_first, int n_v_heads, int v_pitch, int v_offset, int out_pitch,
-                              int out_offset, hipStream_t stream) {
+                              int out_offset, const float* slopes, hipStream_t stream) {
   if (head_dim != DH) return variant_fail(TL_ERR_ARG, "attn_prefill: built for head_dim %d, called with %d", DH, head_dim);
   if (n_tiles < 0 || n_q_heads <= 0 || n_kv_heads <= 0 || page_size <= 0 || bt_stride <= 0 || window < 0 || chunk < 0 || softcap < 0)
     return variant_fail(TL_ERR_ARG, "attn_prefill: bad sizes");
@@ -579,6 +595,7 @@ TL_EXPORT int tl_attn_prefill(const void* q, int q_stride, void* out, int out_st
   if (keep_first < 0 || n_kv_heads % n_v_heads || v_offset < 0 || v_offset + DH > v_pitch || out_offset < 0 || out_offset + DH > out_pitch
       || v_pitch % 8 || v_offset % 8 || out_pitch % 4 || out_offset % 4)
     return variant_fail(TL_ERR_ARG, "attn_prefill: kept keys, value heads or the places of values and outputs do not fit");
+  if (keep_first > 0 && slopes) return variant_fail(TL_ERR_UNSUPPORTED, "attn_prefill: kept first keys together with a bias by distance are not built");
   if (keep_first > 0 && softcap > 0) return variant_fail(TL_ERR_UNSUPPORTED, "attn_prefill: kept first keys together with capped scores are not built");
   const int R = n_q_heads / n_kv_heads;
   if (R > 16) return variant_fail(TL_ERR_UNSUPPORTED, "attn_prefill: %d query heads per kv head exceed 16", R);
@@ -606,21 +623,25 @@ TL_EXPORT int tl_attn_prefill(const void* q, int q_stride, void* out, int out_st
     return variant_fail(TL_ERR_UNSUPPORTED, "attn_prefill: pages of %d tokens are shorter than the %d rows a wave fetches at once at head size %d",
                         page_size, kRowsPerLoad, DH);
   a.scale_log2e = scale * 1.4426950408889634f;
-  a.chunk = chunk; a.sinks = sinks;
+  a.chunk = chunk; a.sinks = sinks; a.slopes = slopes; a.inv_scale = 1.0f / scale;
   a.cap_over_scale = softcap > 0 ? softcap / scale : 0.f;
   a.two_scale_over_cap_log2e = softcap > 0 ? 2.0f * scale / softcap * 1.4426950408889634f : 0.f;
   dim3 grid(n_kv_heads, n_tiles);  // consecutive blocks share a query tile: their loads of q overlap
-  const int mode = softcap > 0 ? 2 : a.keep_first > 0 ? 3 : (window > 0 || chunk > 0) ? 1 : 0;
+  const int mode = slopes ? (softcap > 0 ? 5 : 4) : softcap > 0 ? 2 : a.keep_first > 0 ? 3 : (window > 0 || chunk > 0) ? 1 : 0;
   const int threads = kWaves * kWave;
 #define TL_PREFILL_LAUNCH(rp)                                                                      \
   do {                                                                                             \
     if (key_groups == 2) {                                                                         \
-      if (mode == 2) attn_prefill_kernel<rp, 2, 2><<<grid, 2 * threads, 0, stream>>>(a);           \
+      if (mode == 5) attn_prefill_kernel<rp, 5, 2><<<grid, 2 * threads, 0, stream>>>(a);           \
+      else if (mode == 4) attn_prefill_kernel<rp, 4, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
+      else if (mode == 2) attn_prefill_kernel<rp, 2, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else if (mode == 3) attn_prefill_kernel<rp, 3, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else if (mode == 1) attn_prefill_kernel<rp, 1, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else attn_prefill_kernel<rp, 0, 2><<<grid, 2 * threads, 0, stream>>>(a);                     \
     } else {                                                                                       \
-      if (mode == 2) attn_prefill_kernel<rp, 2, 1><<<grid, threads, 0, stream>>>(a);               \
+      if (mode == 5) attn_prefill_kernel<rp, 5, 1><<<grid, threads, 0, stream>>>(a);               \
+      else if (mode == 4) attn_prefill_kernel<rp, 4, 1><<<grid, threads, 0, stream>>>(a);          \
+      else if (mode == 2) attn_prefill_kernel<rp, 2, 1><<<grid, threads, 0, stream>>>(a);          \
       else if (mode == 3) attn_prefill_kernel<rp, 3, 1><<<grid, threads, 0, stream>>>(a);          \
       else if (mode == 1) attn_prefill_kernel<rp, 1, 1><<<grid, threads, 0, stream>>>(a);          \
       else attn_prefill_kernel<rp, 0, 1><<<grid, threads, 0, stream>>>(a);                         \

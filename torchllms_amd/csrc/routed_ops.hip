@@ -1,6 +1,6 @@
 // Kernels of a routed feed-forward (a mixture of experts whose router's scores are a softmax, with a correction
-// added for the choice only, and whose last outputs may be experts that hand their input through), of a dense
-// feed-forward with biases and the exact gelu, and of layers with a norm on either side of every branch.
+// added for the choice only, and whose last outputs may be experts that hand their input through), of dense
+// feed-forwards (biases and the exact gelu; the squared relu), and of layers with a norm on either side of every branch.
 #include "common.h"
 
 namespace {
@@ -11,14 +11,14 @@ __device__ __forceinline__ float sigmoid_r(float z) { return 1.0f / (1.0f + expf
 // ----------------------------------------------------------------------------- router
 // One wave a token.  z [n, z_stride]: 32-bit router outputs, the first n_out of a row.  s = softmax(z); the `top`
 // largest of s + correction are chosen (of equal ones the lower index), and the weights are their s.
-// correction may be null.  n_groups > 0: the outputs form that many equal groups of neighbours, a group's score is
+// correction may be null, and so may bias, which is added to z first (32-bit).  n_groups > 0: the outputs form that many equal groups of neighbours, a group's score is
 // the largest s in it, and only outputs of the keep_groups best groups (of equal ones the lower) can be chosen.
 // normalize: the weights are divided by their sum (+ 1e-20); then they are multiplied by route_scale.
 constexpr int kRouterPerLane = 8;  // outputs a lane holds: up to 512 experts
 __global__ void __launch_bounds__(256)
 router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __restrict__ correction, int n, int n_out, int top,
                    int32_t* __restrict__ ids, float* __restrict__ weights, int n_groups, int keep_groups, int normalize,
-                   float route_scale) {
+                   float route_scale, const float* __restrict__ bias) {
   const int t = blockIdx.x * (blockDim.x / kWave) + threadIdx.x / kWave;
   const int lane = threadIdx.x % kWave;
   if (t >= n) return;
@@ -28,7 +28,7 @@ router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __res
 #pragma unroll
   for (int u = 0; u < kRouterPerLane; ++u) {
     const int e = lane + u * kWave;
-    s[u] = e < n_out ? zr[e] : -INFINITY;
+    s[u] = e < n_out ? (bias ? zr[e] + bias[e] : zr[e]) : -INFINITY;
     mx = fmaxf(mx, s[u]);
   }
   mx = wave_max(mx);
@@ -460,91 +460,182 @@ weighted_pair_kernel(const T* __restrict__ a, float sa, const T* __restrict__ b,
 }
 
 // ----------------------------------------------------------------------------- a branch's result into the stream, and the next norm
-// stream[r] += y[r] / sqrt(mean(y[r]^2) + eps) * w_post (32-bit, in place), and, where w_next is given,
-// rows[r] = T(stream[r] / sqrt(mean(stream[r]^2) + eps_next) * w_next): the norm behind a branch and the norm before
-// the next one in a single pass over the row, which stays in LDS in between.
-constexpr int kSandwichThreads = 256;
+// stream[r] += y[r] / sqrt(mean(y[r]^2) + eps) * w_post (32-bit, in place), then stream[r] += add where that vector is
+// given, and, where w_next is given, rows[r] = T(stream[r] / sqrt(mean(stream[r]^2) + eps_next) * w_next): the norm
+// behind a branch and the norm before the next one in a single pass over the row, which stays in LDS in between.
+// PAIR: the branch is the sum of two results, each over its own root mean square and times its own weight and factor,
+// y = s_a a / rms(a) w_a + s_b b / rms(b) w_b, worked out in 32-bit.
 template <typename T>
-__global__ void __launch_bounds__(kSandwichThreads)
-post_norm_add_norm_kernel(float* __restrict__ stream, const T* __restrict__ y, const float* __restrict__ w_post, float eps,
-                          const float* __restrict__ w_next, float eps_next, T* __restrict__ rows, int hidden) {
+struct SandwichArgs {
+  float* stream;
+  const T* y;        // the branch (PAIR: the first result, a)
+  const T* b;        // PAIR: the second result
+  const float *w_a, *w_b;
+  float eps_a, s_a, eps_b, s_b;
+  const float* w_post;
+  float eps;
+  const float* w_next;
+  float eps_next;
+  const float* add;
+  T* rows;
+  int hidden;
+};
+
+constexpr int kSandwichThreads = 256;
+template <typename T, bool PAIR>
+__global__ void __launch_bounds__(kSandwichThreads) post_norm_add_norm_kernel(const SandwichArgs<T> g) {
 #pragma clang fp contract(off)
   extern __shared__ __attribute__((aligned(16))) float row_l[];
   __shared__ float scratch[kSandwichThreads / kWave];
+  const int hidden = g.hidden;
+  float* row_b = row_l + hidden;  // (PAIR)
   const size_t r = blockIdx.x;
-  const T* yr = y + r * hidden;
-  float* sr = stream + r * hidden;
-  float ss = 0.f;
+  const T* yr = g.y + r * hidden;
+  float* sr = g.stream + r * hidden;
+  float ss = 0.f, ss_b = 0.f;
   for (int i = threadIdx.x; i < hidden; i += kSandwichThreads) {
     const float v = to_f32(yr[i]);
     row_l[i] = v;
     ss += v * v;
+    if constexpr (PAIR) {
+      const float u = to_f32(g.b[r * hidden + i]);
+      row_b[i] = u;
+      ss_b += u * u;
+    }
   }
   ss = block_sum<kSandwichThreads / kWave>(ss, scratch);
-  const float inv = 1.0f / sqrtf(ss / (float)hidden + eps);
+  if constexpr (PAIR) {
+    ss_b = block_sum<kSandwichThreads / kWave>(ss_b, scratch);
+    const float inv_a = 1.0f / sqrtf(ss / (float)hidden + g.eps_a), inv_b = 1.0f / sqrtf(ss_b / (float)hidden + g.eps_b);
+    ss = 0.f;
+    for (int i = threadIdx.x; i < hidden; i += kSandwichThreads) {
+      const float v = g.s_a * (row_l[i] * inv_a * g.w_a[i]) + g.s_b * (row_b[i] * inv_b * g.w_b[i]);
+      row_l[i] = v;
+      ss += v * v;
+    }
+    ss = block_sum<kSandwichThreads / kWave>(ss, scratch);
+  }
+  const float inv = 1.0f / sqrtf(ss / (float)hidden + g.eps);
   float s2 = 0.f;
   for (int i = threadIdx.x; i < hidden; i += kSandwichThreads) {
-    const float h = sr[i] + row_l[i] * inv * w_post[i];
+    float h = sr[i] + row_l[i] * inv * g.w_post[i];
+    if (g.add) h = h + g.add[i];
     sr[i] = h;
     row_l[i] = h;
     s2 += h * h;
   }
-  if (w_next == nullptr) return;
+  if (g.w_next == nullptr) return;
   s2 = block_sum<kSandwichThreads / kWave>(s2, scratch);
-  const float inv2 = 1.0f / sqrtf(s2 / (float)hidden + eps_next);
-  for (int i = threadIdx.x; i < hidden; i += kSandwichThreads) rows[r * hidden + i] = from_f32<T>(row_l[i] * inv2 * w_next[i]);
+  const float inv2 = 1.0f / sqrtf(s2 / (float)hidden + g.eps_next);
+  for (int i = threadIdx.x; i < hidden; i += kSandwichThreads) g.rows[r * hidden + i] = from_f32<T>(row_l[i] * inv2 * g.w_next[i]);
 }
-
 
 // The same for few rows of up to HELD * 256 elements: a launch is then as long as a row's trips to memory, so everything
 // a thread needs is asked for at once (an element past the end is the row's first once more, and not used).  Operation
 // for operation the kernel above: the same bits.
-template <typename T, int HELD>
-__global__ void __launch_bounds__(kSandwichThreads)
-post_norm_add_norm_held_kernel(float* __restrict__ stream, const T* __restrict__ y, const float* __restrict__ w_post, float eps,
-                               const float* __restrict__ w_next, float eps_next, T* __restrict__ rows, int hidden) {
+template <typename T, int HELD, bool PAIR>
+__global__ void __launch_bounds__(kSandwichThreads) post_norm_add_norm_held_kernel(const SandwichArgs<T> g) {
 #pragma clang fp contract(off)
   __shared__ float scratch[kSandwichThreads / kWave];
+  const int hidden = g.hidden;
   const size_t r = blockIdx.x;
-  const T* yr = y + r * hidden;
-  float* sr = stream + r * hidden;
-  T yraw[HELD];
-  float sv[HELD], wp[HELD], wn[HELD];
+  const T* yr = g.y + r * hidden;
+  float* sr = g.stream + r * hidden;
+  T yraw[HELD], braw[PAIR ? HELD : 1];
+  float sv[HELD], wp[HELD], wn[HELD], av[HELD], wa[PAIR ? HELD : 1], wb[PAIR ? HELD : 1];
 #pragma unroll
   for (int c = 0; c < HELD; ++c) {
     const int i = threadIdx.x + c * kSandwichThreads;
     const int at = i < hidden ? i : 0;
     yraw[c] = yr[at];
     sv[c] = sr[at];
-    wp[c] = w_post[at];
-    wn[c] = w_next ? w_next[at] : 0.f;
+    wp[c] = g.w_post[at];
+    wn[c] = g.w_next ? g.w_next[at] : 0.f;
+    av[c] = g.add ? g.add[at] : 0.f;
+    if constexpr (PAIR) {
+      braw[c] = g.b[r * hidden + at];
+      wa[c] = g.w_a[at];
+      wb[c] = g.w_b[at];
+    }
   }
-  float yv[HELD];
-  float ss = 0.f;
+  float yv[HELD], bv[PAIR ? HELD : 1];
+  float ss = 0.f, ss_b = 0.f;
 #pragma unroll
   for (int c = 0; c < HELD; ++c) {
-    yv[c] = threadIdx.x + c * kSandwichThreads < hidden ? to_f32(yraw[c]) : 0.f;
+    const bool in = threadIdx.x + c * kSandwichThreads < hidden;
+    yv[c] = in ? to_f32(yraw[c]) : 0.f;
     ss += yv[c] * yv[c];
+    if constexpr (PAIR) {
+      bv[c] = in ? to_f32(braw[c]) : 0.f;
+      ss_b += bv[c] * bv[c];
+    }
   }
   ss = block_sum<kSandwichThreads / kWave>(ss, scratch);
-  const float inv = 1.0f / sqrtf(ss / (float)hidden + eps);
+  if constexpr (PAIR) {
+    ss_b = block_sum<kSandwichThreads / kWave>(ss_b, scratch);
+    const float inv_a = 1.0f / sqrtf(ss / (float)hidden + g.eps_a), inv_b = 1.0f / sqrtf(ss_b / (float)hidden + g.eps_b);
+    ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < HELD; ++c) {  // (an element past the end is zero in both)
+      yv[c] = g.s_a * (yv[c] * inv_a * wa[c]) + g.s_b * (bv[c] * inv_b * wb[c]);
+      ss += yv[c] * yv[c];
+    }
+    ss = block_sum<kSandwichThreads / kWave>(ss, scratch);
+  }
+  const float inv = 1.0f / sqrtf(ss / (float)hidden + g.eps);
   float s2 = 0.f;
 #pragma unroll
   for (int c = 0; c < HELD; ++c) {
     const int i = threadIdx.x + c * kSandwichThreads;
     if (i < hidden) {
       sv[c] = sv[c] + yv[c] * inv * wp[c];
+      if (g.add) sv[c] = sv[c] + av[c];
       sr[i] = sv[c];
       s2 += sv[c] * sv[c];
     }
   }
-  if (w_next == nullptr) return;
+  if (g.w_next == nullptr) return;
   s2 = block_sum<kSandwichThreads / kWave>(s2, scratch);
-  const float inv2 = 1.0f / sqrtf(s2 / (float)hidden + eps_next);
+  const float inv2 = 1.0f / sqrtf(s2 / (float)hidden + g.eps_next);
 #pragma unroll
   for (int c = 0; c < HELD; ++c) {
     const int i = threadIdx.x + c * kSandwichThreads;
-    if (i < hidden) rows[r * hidden + i] = from_f32<T>(sv[c] * inv2 * wn[c]);
+    if (i < hidden) g.rows[r * hidden + i] = from_f32<T>(sv[c] * inv2 * wn[c]);
+  }
+}
+
+template <typename T, bool PAIR>
+int launch_sandwich(const SandwichArgs<T>& g, int n, hipStream_t stream) {
+  const size_t lds = (size_t)g.hidden * sizeof(float) * (PAIR ? 2 : 1);
+  const bool few = n <= 2 * tl_device_facts().compute_units;
+  if (few && g.hidden <= 4 * kSandwichThreads)
+    post_norm_add_norm_held_kernel<T, 4, PAIR><<<n, kSandwichThreads, 0, stream>>>(g);
+  else if (few && g.hidden <= 16 * kSandwichThreads)
+    post_norm_add_norm_held_kernel<T, 16, PAIR><<<n, kSandwichThreads, 0, stream>>>(g);
+  else {
+    if (lds + 64 > (size_t)tl_device_facts().lds_bytes)
+      return tl_fail(TL_ERR_UNSUPPORTED, "post_norm_add_norm: rows of %d elements do not fit the LDS", g.hidden);
+    if (lds > 48 * 1024) {
+      hipError_t e = hipFuncSetAttribute((const void*)post_norm_add_norm_kernel<T, PAIR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return tl_fail(TL_ERR_HIP, "post_norm_add_norm: %s", hipGetErrorString(e));
+    }
+    post_norm_add_norm_kernel<T, PAIR><<<n, kSandwichThreads, lds, stream>>>(g);
+  }
+  return tl_check_launch("post_norm_add_norm");
+}
+
+// x[i] <- T(max(x[i], 0)^2) in 32-bit, V elements a thread.
+template <typename T, int V>
+__global__ void __launch_bounds__(256) relu_square_kernel(T* __restrict__ x, size_t total) {
+  struct alignas(V * sizeof(T)) Pack { T e[V]; };
+  for (size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * V; i < total; i += (size_t)gridDim.x * blockDim.x * V) {
+    Pack p = *reinterpret_cast<const Pack*>(x + i);
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      const float z = fmaxf(to_f32(p.e[e]), 0.f);
+      p.e[e] = from_f32<T>(z * z);
+    }
+    *reinterpret_cast<Pack*>(x + i) = p;
   }
 }
 
@@ -552,7 +643,8 @@ post_norm_add_norm_held_kernel(float* __restrict__ stream, const T* __restrict__
 
 // ============================================================================= C interface
 TL_EXPORT int tl_router_topk(const float* z, int z_stride, const float* correction, int n, int n_out, int top, int32_t* ids,
-                             float* weights, int n_groups, int keep_groups, int normalize, float route_scale, hipStream_t stream) {
+                             float* weights, int n_groups, int keep_groups, int normalize, float route_scale, const float* bias,
+                             hipStream_t stream) {
   TL_REQUIRE(n >= 0 && n_out > 0 && top > 0 && top <= n_out && z_stride >= n_out, "router_topk: bad sizes");
   TL_REQUIRE(n_groups >= 0 && (n_groups == 0 || (n_groups <= kWave && n_out % n_groups == 0 && keep_groups > 0 && keep_groups <= n_groups
                                                  && (long long)keep_groups * (n_out / n_groups) >= top)),
@@ -562,7 +654,7 @@ TL_EXPORT int tl_router_topk(const float* z, int z_stride, const float* correcti
   if (n == 0) return TL_OK;
   const int per_block = 256 / kWave;
   router_topk_kernel<<<(n + per_block - 1) / per_block, 256, 0, stream>>>(z, z_stride, correction, n, n_out, top, ids, weights, n_groups,
-                                                                         keep_groups, normalize, route_scale);
+                                                                         keep_groups, normalize, route_scale, bias);
   return tl_check_launch("router_topk");
 }
 
@@ -695,26 +787,48 @@ TL_EXPORT int tl_weighted_pair(const void* a, float sa, const void* b, float sb,
 }
 
 TL_EXPORT int tl_post_norm_add_norm(float* stream_rows, const void* y, const float* w_post, float eps, const float* w_next,
-                                    float eps_next, void* rows, int n, int hidden, int dtype, hipStream_t stream) {
+                                    float eps_next, const float* add, void* rows, int n, int hidden, int dtype, hipStream_t stream) {
   TL_REQUIRE(n >= 0 && hidden > 0, "post_norm_add_norm: bad sizes");
   TL_REQUIRE(w_next == nullptr || rows != nullptr, "post_norm_add_norm: the next norm's rows have nowhere to go");
   if (n == 0) return TL_OK;
-  const size_t lds = (size_t)hidden * sizeof(float);
-  if (lds + 64 > (size_t)tl_device_facts().lds_bytes)
-    return tl_fail(TL_ERR_UNSUPPORTED, "post_norm_add_norm: rows of %d elements do not fit the LDS", hidden);
-  if (dtype != TL_F32 && dtype != TL_BF16) return tl_fail(TL_ERR_ARG, "post_norm_add_norm: unknown dtype %d", dtype);
-  const bool few = n <= 2 * tl_device_facts().compute_units;
-#define TL_SANDWICH(T)                                                                                                         \
-  do {                                                                                                                         \
-    if (few && hidden <= 4 * kSandwichThreads)                                                                                 \
-      post_norm_add_norm_held_kernel<T, 4><<<n, kSandwichThreads, 0, stream>>>(stream_rows, (const T*)y, w_post, eps, w_next, eps_next, (T*)rows, hidden);  \
-    else if (few && hidden <= 16 * kSandwichThreads)                                                                           \
-      post_norm_add_norm_held_kernel<T, 16><<<n, kSandwichThreads, 0, stream>>>(stream_rows, (const T*)y, w_post, eps, w_next, eps_next, (T*)rows, hidden); \
-    else                                                                                                                       \
-      post_norm_add_norm_kernel<T><<<n, kSandwichThreads, lds, stream>>>(stream_rows, (const T*)y, w_post, eps, w_next, eps_next, (T*)rows, hidden);        \
-  } while (0)
-  if (dtype == TL_F32) TL_SANDWICH(float);
-  else TL_SANDWICH(bf16_t);
-#undef TL_SANDWICH
-  return tl_check_launch("post_norm_add_norm");
+  if (dtype == TL_F32)
+    return launch_sandwich<float, false>({stream_rows, (const float*)y, nullptr, nullptr, nullptr, 0.f, 0.f, 0.f, 0.f, w_post, eps, w_next,
+                                          eps_next, add, (float*)rows, hidden}, n, stream);
+  if (dtype == TL_BF16)
+    return launch_sandwich<bf16_t, false>({stream_rows, (const bf16_t*)y, nullptr, nullptr, nullptr, 0.f, 0.f, 0.f, 0.f, w_post, eps, w_next,
+                                           eps_next, add, (bf16_t*)rows, hidden}, n, stream);
+  return tl_fail(TL_ERR_ARG, "post_norm_add_norm: unknown dtype %d", dtype);
+}
+
+TL_EXPORT int tl_pair_norm_add_norm(float* stream_rows, const void* a, const float* w_a, float eps_a, float s_a, const void* b,
+                                    const float* w_b, float eps_b, float s_b, const float* w_post, float eps, const float* w_next,
+                                    float eps_next, const float* add, void* rows, int n, int hidden, int dtype, hipStream_t stream) {
+  TL_REQUIRE(n >= 0 && hidden > 0, "pair_norm_add_norm: bad sizes");
+  TL_REQUIRE(w_next == nullptr || rows != nullptr, "pair_norm_add_norm: the next norm's rows have nowhere to go");
+  if (n == 0) return TL_OK;
+  if (dtype == TL_F32)
+    return launch_sandwich<float, true>({stream_rows, (const float*)a, (const float*)b, w_a, w_b, eps_a, s_a, eps_b, s_b, w_post, eps, w_next,
+                                         eps_next, add, (float*)rows, hidden}, n, stream);
+  if (dtype == TL_BF16)
+    return launch_sandwich<bf16_t, true>({stream_rows, (const bf16_t*)a, (const bf16_t*)b, w_a, w_b, eps_a, s_a, eps_b, s_b, w_post, eps, w_next,
+                                          eps_next, add, (bf16_t*)rows, hidden}, n, stream);
+  return tl_fail(TL_ERR_ARG, "pair_norm_add_norm: unknown dtype %d", dtype);
+}
+
+TL_EXPORT int tl_relu_square(void* x, long long total, int dtype, hipStream_t stream) {
+  TL_REQUIRE(total >= 0, "relu_square: bad size");
+  if (total == 0) return TL_OK;
+  const bool wide = total % 8 == 0 && ((uintptr_t)x % 16) == 0;
+  const long long threads = wide ? total / (dtype == TL_F32 ? 4 : 8) : total;
+  const int blocks = (int)((threads + 255) / 256 < 8192 ? (threads + 255) / 256 : 8192);
+  if (dtype == TL_F32) {
+    if (wide) relu_square_kernel<float, 4><<<blocks, 256, 0, stream>>>((float*)x, (size_t)total);
+    else relu_square_kernel<float, 1><<<blocks, 256, 0, stream>>>((float*)x, (size_t)total);
+  } else if (dtype == TL_BF16) {
+    if (wide) relu_square_kernel<bf16_t, 8><<<blocks, 256, 0, stream>>>((bf16_t*)x, (size_t)total);
+    else relu_square_kernel<bf16_t, 1><<<blocks, 256, 0, stream>>>((bf16_t*)x, (size_t)total);
+  } else {
+    return tl_fail(TL_ERR_ARG, "relu_square: unknown dtype %d", dtype);
+  }
+  return tl_check_launch("relu_square");
 }

@@ -32,6 +32,14 @@ ATTENTION_MAX_HEAD_DIM = 256
 ATTENTION_MAX_KEY_DIM = 1024
 
 
+def _slopes(slopes: Optional[torch.Tensor], n_q_heads: int) -> Optional[int]:
+    """The address of a bias by distance: one 32-bit number per query head, which a (capped) score loses for every
+    position between its key and the query; None: no bias."""
+    if slopes is not None and (not slopes.is_cuda or slopes.dtype != torch.float32 or slopes.numel() != n_q_heads or not slopes.is_contiguous()):
+        raise KernelError(f"attention: slopes must be a contiguous float32 GPU vector of {n_q_heads} entries")
+    return _ptr(slopes)
+
+
 def _generic_arguments(qkv, n_q_heads, n_kv_heads, head_dim, k_pages, v_pages, token_seq, positions, block_table, out,
                        sinks=None, v_head_dim=None, values_in_keys=False, value_offset=0, keep_first=0, value_heads=None):
     """What both launches of the plain kernel ask of their arguments; returns (tokens, page size, out, value head
@@ -91,6 +99,7 @@ def attention_generic(
     value_offset: int = 0,
     keep_first: int = 0,
     value_heads: Optional[int] = None,
+    slopes: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Attention of each token's query heads (the first Hq * dh columns of ``qkv``) over the paged
     keys and values of its request; returns [n, Hq * dv].  ``softcap`` c > 0: scores become
@@ -100,7 +109,8 @@ def attention_generic(
     token's value is ``v_head_dim`` channels of its key row, from ``value_offset`` on (``v_pages`` is ``k_pages``).
     ``keep_first`` n > 0: behind a window a query also sees the first n positions of its request.  ``value_heads``:
     the value pages have fewer heads than the key pages, and key head g reads value head ``g % value_heads``
-    (several score maps over the same values: the key heads of map m are ``m * value_heads ..``)."""
+    (several score maps over the same values: the key heads of map m are ``m * value_heads ..``).  ``slopes``: a bias by
+    distance, one 32-bit number per query head that the capped score loses for every position between key and query."""
     n, page_size, out, v_dim, v_pitch = _generic_arguments(qkv, n_q_heads, n_kv_heads, head_dim, k_pages, v_pages, token_seq,
                                                            positions, block_table, out, sinks, v_head_dim, values_in_keys, value_offset,
                                                            keep_first, value_heads)
@@ -110,7 +120,7 @@ def attention_generic(
             qkv.data_ptr(), qkv.stride(0), out.data_ptr(), out.stride(0), k_pages.data_ptr(), v_at,
             token_seq.data_ptr(), positions.data_ptr(), block_table.data_ptr(), block_table.stride(0), n,
             n_q_heads, n_kv_heads, head_dim, page_size, window, float(scale), float(softcap), int(chunk), _ptr(sinks), v_dim,
-            v_pitch, dtype_code(qkv.dtype), int(keep_first), int(value_heads or 0), _stream(),
+            v_pitch, dtype_code(qkv.dtype), int(keep_first), int(value_heads or 0), _slopes(slopes, n_q_heads), _stream(),
         )
     )
     return out
@@ -140,6 +150,7 @@ def attention_generic_split(
     value_offset: int = 0,
     keep_first: int = 0,
     value_heads: Optional[int] = None,
+    slopes: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """``attention_generic`` for steps with few tokens and long contexts (decode): every block of 64
     keys is computed by a wave of its own and a second kernel joins the blocks in order.  The same
@@ -157,14 +168,14 @@ def attention_generic_split(
             qkv.data_ptr(), qkv.stride(0), out.data_ptr(), out.stride(0), k_pages.data_ptr(), v_at,
             token_seq.data_ptr(), positions.data_ptr(), block_table.data_ptr(), block_table.stride(0), n,
             n_q_heads, n_kv_heads, head_dim, page_size, window, float(scale), float(softcap), int(chunk), _ptr(sinks), v_dim,
-            v_pitch, dtype_code(qkv.dtype), max_blocks, partials.data_ptr(), int(keep_first), int(value_heads or 0), _stream(),
+            v_pitch, dtype_code(qkv.dtype), max_blocks, partials.data_ptr(), int(keep_first), int(value_heads or 0), _slopes(slopes, n_q_heads), _stream(),
         )
     )
     return out
 
 
 _DECODE_SIGNATURES = {
-    "tl_attn_decode": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P],
+    "tl_attn_decode": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P],
 }
 DECODE_HEAD_DIMS = (32, 64, 128, 256)
 _DECODE_BLOCK_KEYS = 64  # keys one block pass covers (4 waves x 16): splits are multiples of it
@@ -251,10 +262,11 @@ def attention_decode(
     keep_first: int = 0,
     value_heads: Optional[int] = None,
     v_offset: int = 0,
+    slopes: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Attention of single-token queries over their requests' pages with the split-KV MFMA kernel.
     ``longest``: an upper bound of any token's visible key range, counted from its 16-aligned first
-    visible key (position + 1 without a window; kept first keys are counted here).  ``softcap``, ``chunk``, ``sinks``: as ``attention_generic``.
+    visible key (position + 1 without a window; kept first keys are counted here).  ``softcap``, ``chunk``, ``sinks``, ``slopes``: as ``attention_generic``.
     ``keep_first``: behind a window a query also sees that many first positions of its request.  ``value_heads``,
     ``v_offset``: the value pages are [pages, value_heads, page, v_pitch] with ``value_heads`` dividing the kv heads
     (key head g reads value head ``g % value_heads``) and rows of ``v_pitch`` >= dh channels, of which this call takes
@@ -304,7 +316,7 @@ def attention_decode(
             token_seq.data_ptr(), positions.data_ptr(), block_table.data_ptr(), block_table.stride(0), n,
             n_q_heads, n_kv_heads, head_dim, page_size, window, float(scale), split_size, n_splits,
             _ptr(ws_o), _ptr(ws_ml), float(softcap), int(chunk), _ptr(sinks), int(keep_first) if (window > 0 or chunk > 0) else 0, v_heads,
-            v_pitch, int(v_offset), v_pitch, int(v_offset), _stream(),
+            v_pitch, int(v_offset), v_pitch, int(v_offset), _slopes(slopes, n_q_heads), _stream(),
         ),
         lib,
         "tl_variant_last_error",
@@ -314,7 +326,7 @@ def attention_decode(
 
 # ----------------------------------------------------------------------------- prefill attention (bfloat16, MFMA)
 _PREFILL_SIGNATURES = {
-    "tl_attn_prefill": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P],
+    "tl_attn_prefill": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P],
 }
 PREFILL_HEAD_DIMS = (32, 64, 128, 256)
 
@@ -415,10 +427,11 @@ def attention_prefill(
     keep_first: int = 0,
     value_heads: Optional[int] = None,
     v_offset: int = 0,
+    slopes: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Causal attention of the rows named by the tile lists (see ``prefill_tiles``) with the MFMA
     prefill kernel.  Token t of ``qkv`` / ``out`` is token t of ``qo_indptr``'s numbering.
-    ``key_groups`` = 2: two sets of waves per block share a tile's keys between them.
+    ``key_groups`` = 2: two sets of waves per block share a tile's keys between them.  ``slopes``: as ``attention_generic``.
     ``keep_first``: behind a window a query also sees that many first positions of its request.  ``value_heads``,
     ``v_offset``: the value pages are [pages, value_heads, page, v_pitch] with ``value_heads`` dividing the kv heads
     (key head g reads value head ``g % value_heads``) and rows of ``v_pitch`` >= dh channels, of which this call takes
@@ -455,7 +468,7 @@ def attention_prefill(
             qo_indptr.data_ptr(), kv_lens.data_ptr(), block_table.data_ptr(), block_table.stride(0),
             tile_row.data_ptr(), tile_q0.data_ptr(), tile_row.numel(), n_q_heads, n_kv_heads, head_dim, page_size,
             window, float(scale), int(key_groups), float(softcap), int(chunk), _ptr(sinks), int(keep_first), v_heads, v_pitch, int(v_offset),
-            v_pitch, int(v_offset), _stream(),
+            v_pitch, int(v_offset), _slopes(slopes, n_q_heads), _stream(),
         ),
         lib,
         "tl_variant_last_error",

@@ -39,6 +39,7 @@ CORE_SOURCES = [
     "head_ops.hip",
     "routed_ops.hip",
     "stream_ops.hip",
+    "retention.hip",
 ]
 HEADERS = ["common.h", "qkv_epilogue.h", "no_alloc.h"]
 

@@ -17,6 +17,7 @@ a module's own helpers and tables stay in the module.
                      exact gelu, the norm behind a branch together with the norm before the next
 ``stream_ops``       several residual streams with their weighted reads and writes, the norm without statistics,
                      the join of differential attention's two maps
+``retention_ops``    retention (linear attention with a constant decay per head)
 ``sampling_ops``     the sampling kernel
 """
 
@@ -130,9 +131,15 @@ from .routed_ops import (  # noqa: F401
     expert_glu_rows,
     expert_pair_products,
     PAIR_PRODUCTS_MOST,
+    pair_norm_add_norm,
     post_norm_add_norm,
+    relu_square_,
     router_topk,
     weighted_pair,
+)
+from .retention_ops import (  # noqa: F401
+    RETENTION_MAX_KEY_DIM,
+    retention,
 )
 from .stream_ops import (  # noqa: F401
     MAX_STREAMS,

@@ -1,7 +1,7 @@
 """Kernels of a routed feed-forward (router with softmax scores and a correction for the choice, the (token, choice)
 pairs gathered in the order of their experts, experts over their rows, experts that hand their input through, a
-shared expert with a gate), of a dense
-feed-forward with biases and the exact gelu, and of layers with a norm on either side of every branch."""
+shared expert with a gate), of dense
+feed-forwards (biases and the exact gelu; the squared relu), and of layers with a norm on either side of every branch."""
 
 from __future__ import annotations
 
@@ -16,18 +16,20 @@ ROUTER_MAX_OUTPUTS = 512
 
 
 def router_topk(z: torch.Tensor, n_out: int, correction: Optional[torch.Tensor], top: int, groups: int = 0, keep_groups: int = 0,
-                normalize: bool = False, scale: float = 1.0) -> Tuple[torch.Tensor, torch.Tensor]:
+                normalize: bool = False, scale: float = 1.0, bias: Optional[torch.Tensor] = None) -> Tuple[torch.Tensor, torch.Tensor]:
     """``z`` float32 [n, >= n_out]: the router's outputs in the first ``n_out`` columns.  ``s = softmax(z)``; the
     ``top`` outputs with the largest ``s + correction`` are chosen (of equal ones the lower index).  Returns
     ``(ids int32 [n, top], weights float32 [n, top])``, the weights being the chosen outputs' ``s``.  ``correction``
     None: the largest ``s``.  ``groups`` g > 0: the outputs form g equal groups of neighbours, a group's score is the
     largest ``s`` in it, and only outputs of the ``keep_groups`` best groups can be chosen.  ``normalize``: the weights
-    are divided by their sum (+ 1e-20); ``scale`` then multiplies them."""
-    _gpu(z, correction)
+    are divided by their sum (+ 1e-20); ``scale`` then multiplies them.  ``bias`` (float32 [n_out]) is added to ``z``
+    first; with ``normalize`` the weights are then the softmax of ``z + bias`` over the chosen outputs alone."""
+    _gpu(z, correction, bias)
     if z.dim() != 2 or z.dtype != torch.float32 or z.stride(1) != 1 or z.shape[1] < n_out:
         raise KernelError(f"router_topk: z must be float32 [n, >= {n_out}] with contiguous rows")
-    if correction is not None and (tuple(correction.shape) != (n_out,) or correction.dtype != torch.float32 or not correction.is_contiguous()):
-        raise KernelError(f"router_topk: correction must be a float32 vector of {n_out} entries")
+    for v in (correction, bias):
+        if v is not None and (tuple(v.shape) != (n_out,) or v.dtype != torch.float32 or not v.is_contiguous()):
+            raise KernelError(f"router_topk: correction and bias must be float32 vectors of {n_out} entries")
     if not 0 < top <= n_out:
         raise KernelError(f"router_topk: {top} choices among {n_out} outputs")
     if groups and (groups < 0 or groups > 64 or n_out % groups or not 0 < keep_groups <= groups or keep_groups * (n_out // groups) < top):
@@ -36,7 +38,7 @@ def router_topk(z: torch.Tensor, n_out: int, correction: Optional[torch.Tensor],
     ids = torch.empty((n, top), dtype=torch.int32, device=z.device)
     weights = torch.empty((n, top), dtype=torch.float32, device=z.device)
     check(core().tl_router_topk(z.data_ptr(), z.stride(0), _ptr(correction), n, n_out, top, ids.data_ptr(), weights.data_ptr(),
-                                int(groups), int(keep_groups), 1 if normalize else 0, float(scale), _stream()))
+                                int(groups), int(keep_groups), 1 if normalize else 0, float(scale), _ptr(bias), _stream()))
     return ids, weights
 
 
@@ -207,20 +209,64 @@ def post_norm_add_norm(
     eps: float,
     next_weight: Optional[torch.Tensor] = None,
     next_eps: float = 0.0,
+    add: Optional[torch.Tensor] = None,
 ) -> Optional[torch.Tensor]:
-    """``stream += branch / rms(branch) * post_weight`` in place and in 32-bit, and, with ``next_weight``, the rows
-    ``stream / rms(stream) * next_weight`` in the branch's dtype: the norm behind a branch and the norm before the next
-    one, one pass over each row.  Both weights are 32-bit vectors (whatever factors a norm has, folded into one)."""
-    _gpu(stream, branch, post_weight, next_weight)
+    """``stream += branch / rms(branch) * post_weight`` in place and in 32-bit, then ``stream += add`` if that vector is
+    given, and, with ``next_weight``, the rows ``stream / rms(stream) * next_weight`` in the branch's dtype: the norm
+    behind a branch and the norm before the next one, one pass over each row.  Weights and ``add`` are 32-bit vectors
+    (whatever factors a norm has, folded into one)."""
+    rows = _sandwich_rows(stream, (branch,), (post_weight, next_weight, add), next_weight is not None)
+    n, hidden = stream.shape
+    check(core().tl_post_norm_add_norm(stream.data_ptr(), branch.data_ptr(), post_weight.data_ptr(), float(eps), _ptr(next_weight),
+                                       float(next_eps), _ptr(add), _ptr(rows), n, hidden, dtype_code(branch.dtype), _stream()))
+    return rows
+
+
+def pair_norm_add_norm(
+    stream: torch.Tensor,
+    a: torch.Tensor,
+    a_weight: torch.Tensor,
+    a_eps: float,
+    a_scale: float,
+    b: torch.Tensor,
+    b_weight: torch.Tensor,
+    b_eps: float,
+    b_scale: float,
+    post_weight: torch.Tensor,
+    eps: float,
+    next_weight: Optional[torch.Tensor] = None,
+    next_eps: float = 0.0,
+    add: Optional[torch.Tensor] = None,
+) -> Optional[torch.Tensor]:
+    """``post_norm_add_norm`` of the branch ``a_scale * a / rms(a) * a_weight + b_scale * b / rms(b) * b_weight``, which
+    is worked out in 32-bit and never leaves the kernel."""
+    rows = _sandwich_rows(stream, (a, b), (a_weight, b_weight, post_weight, next_weight, add), next_weight is not None)
+    n, hidden = stream.shape
+    check(core().tl_pair_norm_add_norm(stream.data_ptr(), a.data_ptr(), a_weight.data_ptr(), float(a_eps), float(a_scale), b.data_ptr(),
+                                       b_weight.data_ptr(), float(b_eps), float(b_scale), post_weight.data_ptr(), float(eps),
+                                       _ptr(next_weight), float(next_eps), _ptr(add), _ptr(rows), n, hidden, dtype_code(a.dtype), _stream()))
+    return rows
+
+
+def _sandwich_rows(stream, branches, vectors, want_rows: bool) -> Optional[torch.Tensor]:
+    """What both launches ask of their arguments; returns the tensor for the next norm's rows, if there is one."""
+    _gpu(stream, *branches, *vectors)
     if stream.dim() != 2 or stream.dtype != torch.float32 or not stream.is_contiguous():
         raise KernelError("post_norm_add_norm: the stream must be a contiguous float32 matrix")
     n, hidden = stream.shape
-    if tuple(branch.shape) != (n, hidden) or not branch.is_contiguous():
-        raise KernelError("post_norm_add_norm: the branch must be contiguous and of the stream's shape")
-    for w in (post_weight, next_weight):
+    for branch in branches:
+        if tuple(branch.shape) != (n, hidden) or not branch.is_contiguous() or branch.dtype != branches[0].dtype:
+            raise KernelError("post_norm_add_norm: the branch must be contiguous, of the stream's shape and of one dtype")
+    for w in vectors:
         if w is not None and (tuple(w.shape) != (hidden,) or w.dtype != torch.float32 or not w.is_contiguous()):
             raise KernelError(f"post_norm_add_norm: weights must be float32 vectors of {hidden} entries")
-    rows = torch.empty_like(branch) if next_weight is not None else None
-    check(core().tl_post_norm_add_norm(stream.data_ptr(), branch.data_ptr(), post_weight.data_ptr(), float(eps), _ptr(next_weight),
-                                       float(next_eps), _ptr(rows), n, hidden, dtype_code(branch.dtype), _stream()))
-    return rows
+    return torch.empty_like(branches[0]) if want_rows else None
+
+
+def relu_square_(x: torch.Tensor) -> torch.Tensor:
+    """``max(x, 0)^2`` element by element, in 32-bit, rounded once to x's dtype; in place."""
+    _gpu(x)
+    if not x.is_contiguous():
+        raise KernelError("relu_square_: x must be contiguous")
+    check(core().tl_relu_square(x.data_ptr(), x.numel(), dtype_code(x.dtype), _stream()))
+    return x

@@ -3,7 +3,7 @@
 from __future__ import annotations
 
 import logging
-from typing import Dict, Optional
+from typing import Dict, Optional, Sequence
 
 import torch
 
@@ -49,6 +49,9 @@ class Attention(Mixer):
 
     ``keep_first`` n > 0 (with a window): a query also sees the first n positions of its request, at their true
     positions; their pages are never given back.
+
+    ``slopes``: a bias by distance: one number per query head, and head h's (capped) score loses ``slopes[h] * (i - j)``
+    between the query at position i and the key at position j.
     """
 
     #: every launch is fixed by the step's shape: a decode step may be recorded in a HIP graph
@@ -80,6 +83,7 @@ class Attention(Mixer):
         out_gate: Optional[str] = None,
         values_from_keys: bool = False,
         keep_first: int = 0,
+        slopes: Optional[Sequence[float]] = None,
     ):
         self.values_from_keys = bool(values_from_keys)
         self.keep_first = int(keep_first)
@@ -105,6 +109,10 @@ class Attention(Mixer):
         self.has_sinks = bool(sinks)
         if self.qk_norm_eps < 0 or self.softcap < 0 or self.chunk < 0:
             raise ValueError("attention: qk_norm_eps, softcap and chunk must not be negative")
+        if slopes is not None and len(slopes) != num_heads:
+            raise ValueError(f"attention: {len(slopes)} slopes for {num_heads} heads")
+        self.slope_values = None if slopes is None else [float(v) for v in slopes]
+        self.slopes: Optional[torch.Tensor] = None
         self.qk_norm_weight = bool(qk_norm_weight)
         self.q_temp_coef = float(q_temp_coef)
         self.q_temp_every = int(q_temp_every)
@@ -142,7 +150,8 @@ class Attention(Mixer):
     @property
     def extended(self) -> bool:
         """Whether the layer needs what only the unfused path and the plain attention kernel do."""
-        return (self.v_head_dim != self.head_dim or self.qk_norm_eps > 0 or self.softcap > 0 or self.chunk > 0 or self.has_sinks)
+        return (self.v_head_dim != self.head_dim or self.qk_norm_eps > 0 or self.softcap > 0 or self.chunk > 0 or self.has_sinks
+                or self.slope_values is not None)
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         q = self.num_heads * self.head_dim
@@ -219,6 +228,8 @@ class Attention(Mixer):
         self.wo = tensors["wo.weight"].contiguous()
         if self.has_sinks:
             self.sinks = tensors["sinks"].float().contiguous()
+        if self.slope_values is not None:
+            self.slopes = torch.tensor(self.slope_values, dtype=torch.float64).float().to(self.wo.device)
         self.position.to(self.wo.device)
 
     def linear_weights(self):
@@ -276,7 +287,7 @@ class Attention(Mixer):
         attn = paged_attention(
             qkv, self.num_heads, self.num_kv_heads, self.head_dim, cache.k_pages, cache.v_pages, ctx, g, self.window,
             self.softmax_scale, softcap=self.softcap, chunk=self.chunk, sinks=self.sinks, v_head_dim=self.v_head_dim,
-            keep_first=self.keep_first,
+            keep_first=self.keep_first, slopes=self.slopes,
         )
         return ops.linear_to_sum(attn, self.wo, may_wait=True)
 
@@ -307,6 +318,7 @@ class Attention(Mixer):
         attn = paged_attention(
             rows, H, self.num_kv_heads, dk, cache.k_pages, cache.v_pages, ctx, g, self.window, self.softmax_scale,
             softcap=self.softcap, chunk=self.chunk, sinks=self.sinks, v_head_dim=dv, keep_first=self.keep_first,
+            slopes=self.slopes,
         )
         if self.out_gate is not None:
             gate_at = v_at + n_kv_in_row * dv

@@ -189,6 +189,22 @@ class Mixer(Part):
         raise NotImplementedError
 
 
+class Following:
+    """What comes right after a layer's run in the order of execution: ``block``, the arrangement that runs next (None
+    behind the last one), and ``vector``, a 32-bit vector that is added to the residual stream before it (or None).
+    The model leaves it in the step's scratch before every run.  An arrangement that adds the vector itself (its last
+    kernel has the rows in hand) takes it with ``take_vector``; what is left there the model adds."""
+
+    KEY = "following"
+
+    def __init__(self, block: Optional["Block"], vector: Optional[torch.Tensor] = None):
+        self.block, self.vector = block, vector
+
+    def take_vector(self) -> Optional[torch.Tensor]:
+        vector, self.vector = self.vector, None
+        return vector
+
+
 class Block(Part):
     """Arrangement of one layer's parts.  ``SLOTS`` names the sub-parts the arrangement has and the
     kind of each ("mixer", "feed_forward" or "norm"), in the order their tensors are listed; the
@@ -232,10 +248,10 @@ class Block(Part):
             prefix = slot + "."
             part.bind({k[len(prefix):]: v for k, v in tensors.items() if k.startswith(prefix)})
 
-    def expects(self, following: Optional["Block"]) -> None:
-        """Told once, when the model is put together: the arrangement that runs right after this one in every run of
-        this layer (None: the last layer, or a layer whose runs are followed by different arrangements).  An
-        arrangement may leave work to, or do work for, the one that follows; the default does neither."""
+    @staticmethod
+    def following(ctx) -> "Following":
+        """What comes after the run that is at work: an arrangement may leave work to, or do work for, what follows."""
+        return ctx.scratch.get(Following.KEY) or Following(None)
 
     def forward(self, h, delta, ctx, cache):
         raise NotImplementedError

@@ -2,7 +2,7 @@
 
 from __future__ import annotations
 
-from typing import Dict, Optional
+from typing import Dict
 
 import torch
 
@@ -126,23 +126,15 @@ class BranchNormMixerBlock(_BranchNorm):
 class _Sandwich(Block):
     """Layers with a norm before and a norm behind every branch, over a 32-bit residual stream:
     ``x <- x + post(branch(pre(x)))``, one branch after the other.  The norm behind a branch and the norm before the
-    next one (of this layer or of the next layer of this kind) run as one kernel over the rows: a layer hands the
-    rows that the next layer's first norm would make on, under ``_ROWS`` of the step's scratch, when the next layer
-    has said (``expects``) which norm that is."""
+    next one (of this layer or of the layer that runs next, if it is of this kind) run as one kernel over the rows; a
+    step vector that comes between two runs is added on the way.  A layer hands the rows that the next layer's first
+    norm would make on, under ``_ROWS`` of the step's scratch."""
 
     graph_safe = True
     _ROWS = "sandwich_rows"  # in ctx.scratch: (the stream the rows were made from, the norm that made them, the rows)
 
     def first_norm(self):
         return self.norm1
-
-    def __init__(self, parts):
-        super().__init__(parts)
-        self.next_first_norm = None  # the first norm of the layer that runs after this one, if that is known
-
-    def expects(self, following: "Block") -> None:
-        """Told once, when the model is put together: ``following`` runs right after this layer."""
-        self.next_first_norm = following.first_norm() if isinstance(following, _Sandwich) else None
 
     def rows_for(self, norm, h, ctx):
         kept = ctx.scratch.get(self._ROWS)
@@ -153,16 +145,21 @@ class _Sandwich(Block):
     def mix_branch(self, y, ctx, cache):
         raise NotImplementedError
 
+    def close_mixer(self, h, branch, then, add=None):
+        """The mixer's branch into the stream: ``(stream, what the norm `then` makes of it)``."""
+        return self.norm1b.forward_branch_then(h, branch, then, add=add)
+
     def forward(self, h, delta, ctx, cache):
         if delta is not None:
             h = h + ops.resolved(delta).float()
         a = self.mix_branch(self.rows_for(self.norm1, h, ctx), ctx, cache)
-        has_mlp = "mlp" in self.parts
-        after = self.norm2 if has_mlp else self.next_first_norm
-        h, y = self.norm1b.forward_branch_then(h, a, after)
-        if has_mlp:
-            after = self.next_first_norm
-            h, y = self.norm2b.forward_branch_then(h, self.mlp.forward(y, ctx), after)
+        following = self.following(ctx)
+        after = following.block.first_norm() if isinstance(following.block, _Sandwich) else None
+        if "mlp" in self.parts:
+            h, y = self.close_mixer(h, a, self.norm2)
+            h, y = self.norm2b.forward_branch_then(h, self.mlp.forward(y, ctx), after, add=following.take_vector())
+        else:
+            h, y = self.close_mixer(h, a, after, add=following.take_vector())
         if after is not None:
             ctx.scratch[self._ROWS] = (h, after, y)
         return h, None
@@ -217,6 +214,35 @@ class SandwichPairMixerBlock(_SandwichPair):
     SLOTS = {"norm1": "norm", "left": "mixer", "right": "mixer", "norm1b": "norm"}
 
 
+class _SandwichNormedPair(_SandwichPair):
+    """Two mixers side by side whose results are normed each by a norm of its own before they are weighted and added:
+    the branch is ``left_scale * left_out(left(h)) + right_scale * right_out(right(h))``.  Both norms, the sum, the
+    norm behind the branch, the stream's sum and the next norm are one kernel over the rows."""
+
+    def mix_branch(self, y, ctx, cache):
+        a = ops.resolved(self.left.forward(y, ctx, cache["left"]))
+        b = ops.resolved(self.right.forward(y, ctx, cache["right"]))
+        return (a, self.left_out, self.left_scale), (b, self.right_out, self.right_scale)
+
+    def close_mixer(self, h, branch, then, add=None):
+        return self.norm1b.forward_pair_then(h, branch[0], branch[1], then, add=add)
+
+
+@BLOCKS.register("sandwich_normed_pair")
+class SandwichNormedPairBlock(_SandwichNormedPair):
+    """``x <- x + norm1b(s_l left_out(left(norm1(x))) + s_r right_out(right(norm1(x)))); x <- x + norm2b(mlp(norm2(x)))``."""
+
+    SLOTS = {"norm1": "norm", "left": "mixer", "right": "mixer", "left_out": "norm", "right_out": "norm", "norm1b": "norm",
+             "norm2": "norm", "mlp": "feed_forward", "norm2b": "norm"}
+
+
+@BLOCKS.register("sandwich_normed_pair_mixer")
+class SandwichNormedPairMixerBlock(_SandwichNormedPair):
+    """The same layer without a feed-forward."""
+
+    SLOTS = {"norm1": "norm", "left": "mixer", "right": "mixer", "left_out": "norm", "right_out": "norm", "norm1b": "norm"}
+
+
 class _Hyper(Block):
     """Layers over several residual streams (hyper-connections).  Instead of one stream there are ``streams`` 32-bit
     copies ``x_1 .. x_S`` (all equal to the embedding's rows when the first such layer opens them).  Sublayer q
@@ -224,7 +250,7 @@ class _Hyper(Block):
     back into all streams at once, ``x_r <- sum_s mix_q[s, r] x_s + out_q[r] y``: the tensors ``hc<q>.in`` [S],
     ``hc<q>.out`` [S] and ``hc<q>.mix`` [S, S] (indexed [from, to]) are the arrangement's own.  A sublayer's write, the
     next sublayer's read and its norm are one kernel over the rows (also across layers, when the next layer is of
-    this kind: ``expects``).  The norms take several streams (``dynamic_tanh``); whoever reads the model's last
+    this kind).  The norms take several streams (``dynamic_tanh``); whoever reads the model's last
     streams (the final norm) takes their plain sum."""
 
     graph_safe = True
@@ -237,7 +263,6 @@ class _Hyper(Block):
         self.streams = streams
         self.has_mlp = "mlp" in self.parts
         self.hc: Dict[str, torch.Tensor] = {}
-        self.next_block: Optional["_Hyper"] = None
 
     def own_specs(self) -> Dict[str, ParamSpec]:
         S, specs = self.streams, {}
@@ -255,9 +280,6 @@ class _Hyper(Block):
     def bind(self, tensors) -> None:
         super().bind(tensors)
         self.hc = {name: tensors[name].float().contiguous() for name in self.own_specs()}
-
-    def expects(self, following) -> None:
-        self.next_block = following if isinstance(following, _Hyper) and following.streams == self.streams else None
 
     def mix_branch(self, y, ctx, cache):
         raise NotImplementedError
@@ -279,8 +301,8 @@ class _Hyper(Block):
         if self.has_mlp:
             y = self.norm2.read(h, self.hc["hc2.in"], branch=a, mix=mix, out_weights=out)
             last, mix, out = ops.resolved(self.mlp.forward(y, ctx)), self.hc["hc2.mix"], self.hc["hc2.out"]
-        nxt = self.next_block
-        if nxt is not None:
+        nxt = self.following(ctx).block
+        if isinstance(nxt, _Hyper) and nxt.streams == self.streams:
             y = nxt.norm1.read(h, nxt.hc["hc1.in"], branch=last, mix=mix, out_weights=out)
             ctx.scratch[self._ROWS] = (h, nxt.norm1, y)
         else:

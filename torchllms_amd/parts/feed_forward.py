@@ -70,6 +70,30 @@ class DenseGelu(FeedForward):
         return ops.add_bias_(ops.linear(mid, self.w_down), self.b_down)
 
 
+@FEED_FORWARDS.register("dense_relu2")
+class DenseReluSquare(FeedForward):
+    """``W_down max(W_up x, 0)^2``, no biases."""
+
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int):
+        self.hidden_size, self.intermediate_size = hidden_size, intermediate_size
+        self.w_up = self.w_down = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        f, d = self.intermediate_size, self.hidden_size
+        return {"up.weight": ParamSpec((f, d)), "down.weight": ParamSpec((d, f))}
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.w_up, self.w_down = tensors["up.weight"].contiguous(), tensors["down.weight"].contiguous()
+
+    def linear_weights(self):
+        return [self.w_up, (self.w_down, "sum")]
+
+    def forward(self, x, ctx):
+        return ops.linear_to_sum(ops.relu_square_(ops.linear(ops.resolved(x), self.w_up)), self.w_down)
+
+
 @FEED_FORWARDS.register("routed")
 class RoutedExperts(FeedForward):
     """A mixture of ``num_experts`` gated feed-forwards ``W_down (silu(W_gate x) * (W_up x))`` without biases, of which
@@ -81,7 +105,8 @@ class RoutedExperts(FeedForward):
     ``correction`` False: there is no correction, the largest scores are chosen.  ``groups`` g > 0 with ``keep_groups``:
     the experts form g equal groups of neighbours, a group's score is the largest score in it, and only experts of
     the best ``keep_groups`` groups can be chosen.  ``normalize``: the chosen scores are divided by their sum
-    (+ 1e-20); ``route_scale`` then multiplies them.
+    (+ 1e-20); ``route_scale`` then multiplies them.  ``router_bias``: a vector (tensor ``router.bias``) is added to the
+    router's outputs; with ``normalize`` the weights are the softmax of the chosen outputs alone.
 
     A token's result depends on nothing but the token.  The (token, choice) pairs of a step are put in the order of
     their experts on the device, and a kernel walks every expert's rows with the expert's weights read once for eight
@@ -98,7 +123,7 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, num_identity: int = 0, shared_size: int = 0,
                  shared_gate: bool = True, correction: bool = True, groups: int = 0, keep_groups: int = 0, normalize: bool = False,
-                 route_scale: float = 1.0):
+                 route_scale: float = 1.0, router_bias: bool = False):
         for name, v in (("expert_size", expert_size), ("num_experts", num_experts), ("top", top)):
             if not isinstance(v, int) or v <= 0:
                 raise ValueError(f"routed: {name} must be a positive integer, got {v!r}")
@@ -106,6 +131,7 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed: {top} choices among {num_experts} + {num_identity} outputs; sizes must not be negative")
         self.hidden_size, self.F, self.E, self.I, self.top, self.shared = hidden_size, expert_size, num_experts, num_identity, top, shared_size
         self.shared_gate, self.has_correction = bool(shared_gate) and shared_size > 0, bool(correction)
+        self.has_router_bias, self.router_bias = bool(router_bias), None
         self.groups, self.keep_groups, self.normalize, self.route_scale = int(groups or 0), int(keep_groups or 0), bool(normalize), float(route_scale)
         n_out = num_experts + num_identity
         if self.groups and (self.groups < 0 or n_out % self.groups or not 0 < self.keep_groups <= self.groups
@@ -119,6 +145,8 @@ class RoutedExperts(FeedForward):
         specs = {"router.weight": ParamSpec((n, d), init="wide")}
         if self.has_correction:
             specs["correction"] = ParamSpec((n,), init="zeros")
+        if self.has_router_bias:
+            specs["router.bias"] = ParamSpec((n,), init="zeros")
         for e in range(self.E):
             specs[f"experts.{e}.w1.weight"] = ParamSpec((f, d))
             specs[f"experts.{e}.w3.weight"] = ParamSpec((f, d))
@@ -145,6 +173,7 @@ class RoutedExperts(FeedForward):
         rows = [tensors["router.weight"]] + ([tensors["shared.gate.weight"]] if self.shared_gate else [])
         self.w_router = torch.cat(rows, dim=0).contiguous()
         self.correction = tensors["correction"].float().contiguous() if self.has_correction else None
+        self.router_bias = tensors["router.bias"].float().contiguous() if self.has_router_bias else None
         self.w_gu = torch.stack([torch.cat([tensors[f"experts.{e}.w1.weight"], tensors[f"experts.{e}.w3.weight"]], dim=0)
                                  for e in range(self.E)]).contiguous()
         self.w_down = torch.stack([tensors[f"experts.{e}.w2.weight"] for e in range(self.E)]).contiguous()
@@ -167,7 +196,7 @@ class RoutedExperts(FeedForward):
         n_out = self.E + self.I
         z = ops.linear(x, self.w_router, out_dtype=torch.float32)
         ids, weights = ops.router_topk(z, n_out, self.correction, self.top, groups=self.groups, keep_groups=self.keep_groups,
-                                       normalize=self.normalize, scale=self.route_scale)
+                                       normalize=self.normalize, scale=self.route_scale, bias=self.router_bias)
         shared = gate = None
         if self.shared:
             shared = ops.linear(ops.linear_glu(x, self.shared_w13), self.shared_w2)

@@ -2,12 +2,13 @@
 
 from __future__ import annotations
 
-from typing import Dict, List, Tuple
+from typing import Dict, List, Optional, Tuple
 
 import torch
 
 from ..config.spec import ModelSpec
-from .base import BLOCKS, EMBEDDINGS, HEADS, NORMS, SLOT_KINDS, Block, ParamSpec, Part
+from ..kernels import ops
+from .base import BLOCKS, EMBEDDINGS, HEADS, NORMS, SLOT_KINDS, Block, Following, ParamSpec, Part
 
 # importing the modules registers the built-in parts
 from . import attention as _attention  # noqa: F401
@@ -25,7 +26,8 @@ class Model:
 
     Tensor names: ``embed.<tensor>``, ``<layer name>.<slot>.<tensor>`` with the slots of the layer's
     block arrangement (``mixer_norm``, ``mixer``, ``ffn_norm``, ``ffn`` for a pre-norm block), then
-    ``final_norm.<tensor>`` and ``head.<tensor>``.
+    ``final_norm.<tensor>`` and ``head.<tensor>``; a model whose order names step vectors has them in
+    ``loop.step`` [vectors, hidden].
     """
 
     def __init__(self, spec: ModelSpec):
@@ -48,14 +50,7 @@ class Model:
             self.blocks.append(block_cls(parts, **layer.block_params))
         self.final_norm = NORMS.build(spec.final_norm)
         self.head = HEADS.build(spec.head)
-        # every arrangement learns which one follows it, where that is the same in all of its runs
-        followers: Dict[int, set] = {}
-        for pos, run in enumerate(spec.order):
-            nxt = spec.order[pos + 1].layer if pos + 1 < len(spec.order) else None
-            followers.setdefault(run.layer, set()).add(nxt)
-        for layer, nexts in followers.items():
-            only = next(iter(nexts)) if len(nexts) == 1 else None
-            self.blocks[layer].expects(self.blocks[only] if only is not None else None)
+        self.step_vectors: Optional[torch.Tensor] = None
         # per run: (slot of a mixer, name of one of the things it keeps or None, key of the cache entry, whether the run owns the entry)
         self._run_caches: List[List[tuple]] = []
         for run_id, run in enumerate(spec.order):
@@ -102,6 +97,8 @@ class Model:
         for layer, block in zip(self.spec.layers, self.blocks):
             for name, spec in block.param_specs().items():
                 out[f"{layer.name}.{name}"] = spec
+        if self.spec.step_vectors:
+            out["loop.step"] = ParamSpec((self.spec.step_vectors, self.spec.hidden_size))
         for name, spec in self.final_norm.param_specs().items():
             out[f"final_norm.{name}"] = spec
         for name, spec in self.head.param_specs().items():
@@ -118,6 +115,8 @@ class Model:
         self.embedding.bind(sub("embed"))
         for layer, block in zip(self.spec.layers, self.blocks):
             block.bind(sub(layer.name))
+        if self.spec.step_vectors:
+            self.step_vectors = tensors["loop.step"].float().contiguous()
         self.final_norm.bind(sub("final_norm"))
         self.head.bind(sub("head"))
         if getattr(self.head, "tied", False):
@@ -166,11 +165,31 @@ class Model:
         return needs
 
     # ------------------------------------------------------------------ one step
+    def _step_vector(self, run) -> Optional[torch.Tensor]:
+        return None if run.step_vector is None else self.step_vectors[run.step_vector]
+
+    @staticmethod
+    def _add_step_vector(h, delta, vector):
+        """The stream with a vector added to every row (a new tensor: what others keep of the old one stays theirs)."""
+        if vector is None:
+            return h, delta
+        if h.dim() != 2:
+            raise ValueError("a step vector is added to one residual stream, not to several")
+        if delta is not None:
+            h = h + ops.resolved(delta).to(h.dtype)
+        return (h.float() + vector).to(h.dtype), None
+
     def forward(self, ctx, cache) -> torch.Tensor:
         """Run this step's tokens; returns float32 logits [len(ctx.logit_rows), vocab]."""
         h = self.embedding.forward(ctx.tokens)
         delta = None
-        for run, entries in zip(self.spec.order, self._run_caches):
+        order = self.spec.order
+        if order:
+            h, delta = self._add_step_vector(h, delta, self._step_vector(order[0]))
+        for pos, (run, entries) in enumerate(zip(order, self._run_caches)):
+            nxt = order[pos + 1] if pos + 1 < len(order) else None
+            following = Following(self.blocks[nxt.layer], self._step_vector(nxt)) if nxt is not None else Following(None)
+            ctx.scratch[Following.KEY] = following
             views = {}
             for slot, name, key, writes in entries:
                 if name is None:
@@ -178,6 +197,7 @@ class Model:
                 else:
                     views.setdefault(slot, {})[name] = cache.view(key, writes)
             h, delta = self.blocks[run.layer].forward(h, delta, ctx, views)
+            h, delta = self._add_step_vector(h, delta, following.take_vector())
         if ctx.logit_rows.numel() == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=h.device)
         x = self.final_norm.forward_rows(h, self.final_norm.delta(delta), ctx.logit_rows)

@@ -71,14 +71,27 @@ class RMSNorm(Norm):
         """Beside a 32-bit stream: the 32-bit vector a normed row is multiplied by (offset and scale folded in)."""
         return self.weight
 
-    def forward_branch_then(self, stream: torch.Tensor, branch, then: Optional["RMSNorm"]):
-        """``stream += norm(branch)`` in place, and ``then.forward(stream)`` of the new stream from the same pass
-        over the rows (None when ``then`` is None: nobody reads them).  Returns ``(stream, rows)``."""
-        if self.stream_dtype is None or (then is not None and (not isinstance(then, RMSNorm) or then.stream_dtype is None)):
-            raise ValueError("rmsnorm: forward_branch_then joins two RMS norms beside the 32-bit residual stream")
+    def forward_branch_then(self, stream: torch.Tensor, branch, then: Optional["RMSNorm"], add: Optional[torch.Tensor] = None):
+        """``stream += norm(branch)`` in place (and ``stream += add``, a 32-bit vector, if one is given), and
+        ``then.forward(stream)`` of the new stream from the same pass over the rows (None when ``then`` is None: nobody
+        reads them).  Returns ``(stream, rows)``."""
+        self._beside_stream(then)
         rows = ops.post_norm_add_norm(stream, ops.resolved(branch), self.weight, self.eps,
-                                      then.weight if then is not None else None, then.eps if then is not None else 0.0)
+                                      then.weight if then is not None else None, then.eps if then is not None else 0.0, add=add)
         return stream, rows
+
+    def forward_pair_then(self, stream: torch.Tensor, left, right, then: Optional["RMSNorm"], add: Optional[torch.Tensor] = None):
+        """``forward_branch_then`` of a branch that is the sum of two results, each normed first: ``left`` and ``right``
+        are ``(rows, norm, factor)``, and the branch is ``sum of factor * norm(rows)``.  One pass over the rows."""
+        self._beside_stream(then, left[1], right[1])
+        (a, norm_a, s_a), (b, norm_b, s_b) = left, right
+        rows = ops.pair_norm_add_norm(stream, a, norm_a.weight, norm_a.eps, s_a, b, norm_b.weight, norm_b.eps, s_b, self.weight, self.eps,
+                                      then.weight if then is not None else None, then.eps if then is not None else 0.0, add=add)
+        return stream, rows
+
+    def _beside_stream(self, *others) -> None:
+        if any(n is not None and (not isinstance(n, RMSNorm) or n.stream_dtype is None) for n in (self,) + others):
+            raise ValueError("rmsnorm: joins RMS norms beside the 32-bit residual stream alone")
 
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         if self.stream_dtype is not None:

@@ -8,12 +8,14 @@ cut into steps anywhere and batched with anything."""
 
 from __future__ import annotations
 
-from typing import Dict, Optional
+from typing import Dict, Optional, Sequence
 
 import torch
 
+from ..config.spec import PartSpec
 from ..kernels import ops
-from .base import MIXERS, Mixer, ParamSpec, StateNeed
+from .base import MIXERS, POSITIONS, Mixer, ParamSpec, StateNeed
+from .positions import step_table
 
 
 @MIXERS.register("selective_scan")
@@ -314,4 +316,61 @@ class GatedLinearAttention(Mixer):
         pre = ops.linear(proj[:, c + v : c + v + self.rank], self.w_a2, out_dtype=torch.float32)
         y = ops.gated_linear(proj[:, :c], pre, self.a_bias, 1.0 / self.tau, proj, c, self.norm_w, self.norm_eps, cache.tensor, 0,
                              ctx.qo_indptr, ctx.slot_ids, self.H, self.dk, self.dv)
+        return ops.linear_to_sum(y, self.w_o)
+
+
+@MIXERS.register("retention")
+class Retention(Mixer):
+    """Retention: linear attention whose state fades by a constant per head.  ``q`` and ``k`` (``num_heads`` heads of
+    ``head_dim``) and ``v`` (heads of ``v_head_dim``) are projections of the input; q and k are rotated (``position``:
+    half pairing, all or the first channels of a head, or none), k is then multiplied by head_dim^-1/2.  Per head the
+    state, zero at the start, goes ``S <- decay_h S + k v^T`` and ``o = S^T q``; o is divided by its root mean square
+    over v_head_dim, multiplied by ``silu(W_g h)`` and projected by W_o.  Rotated queries and keys, decays, the state and
+    the norm are 32-bit."""
+
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, num_heads: int, head_dim: int, v_head_dim: int, decay: Sequence[float], norm_eps: float,
+                 position: PartSpec):
+        for name, v in (("num_heads", num_heads), ("head_dim", head_dim), ("v_head_dim", v_head_dim)):
+            if not isinstance(v, int) or v <= 0:
+                raise ValueError(f"retention: {name} must be a positive integer, got {v!r}")
+        if len(decay) != num_heads:
+            raise ValueError(f"retention: {len(decay)} decays for {num_heads} heads")
+        self.hidden_size, self.H, self.dk, self.dv = hidden_size, num_heads, head_dim, v_head_dim
+        self.decay_values, self.norm_eps = [float(v) for v in decay], float(norm_eps)
+        self.position = POSITIONS.build(position)
+        self.w_all = self.w_o = self.decay = None
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        d, qk, v = self.hidden_size, self.H * self.dk, self.H * self.dv
+        return {"q": ParamSpec((qk, d)), "k": ParamSpec((qk, d)), "v": ParamSpec((v, d)), "g": ParamSpec((v, d)), "o": ParamSpec((d, v))}
+
+    def check_sizes(self, dtype: torch.dtype) -> None:
+        if self.dk > ops.RETENTION_MAX_KEY_DIM:
+            raise ValueError(f"retention: keys of {self.dk} channels; the kernel takes up to {ops.RETENTION_MAX_KEY_DIM} (values: any number)")
+        rotated = getattr(self.position, "rotary_dim", 0)
+        if rotated % 2 or rotated > self.dk or getattr(self.position, "pairing", "half") != "half":
+            raise ValueError(f"retention: {rotated} rotated channels of a head of {self.dk} (even, at most the head size, half pairing)")
+
+    def cache_need(self):
+        return StateNeed(shape=(self.H * self.dv * self.dk,), dtype="float32")
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        # one projection [q | k | v | gate]: a single product per step
+        self.w_all = torch.cat([tensors[n] for n in ("q", "k", "v", "g")], dim=0).contiguous()
+        self.w_o = tensors["o"].contiguous()
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float64).float().to(self.w_o.device)
+        self.position.to(self.w_o.device)
+
+    def linear_weights(self):
+        return [self.w_all, (self.w_o, "sum")]
+
+    def forward(self, x, ctx, cache):
+        qk, v = self.H * self.dk, self.H * self.dv
+        rot = self.position.rotary_args()
+        table = step_table(rot, ctx) if rot is not None and rot.rotary_dim > 0 else None
+        proj = ops.linear(ops.resolved(x), self.w_all)
+        y = ops.retention(proj, 0, qk, 2 * qk, 2 * qk + v, table, rot.rotary_dim if table is not None else 0, self.decay, self.norm_eps,
+                          cache.tensor, 0, ctx.qo_indptr, ctx.slot_ids, self.H, self.dk, self.dv)
         return ops.linear_to_sum(y, self.w_o)

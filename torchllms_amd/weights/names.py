@@ -265,3 +265,31 @@ def nosuzen_name_rules(cfg) -> List[NameRule]:
             rules += [NameRule(p + "left." + ext, f"l{i}.left." + own) for ext, own in left.items()]
             rules += [NameRule(p + "right." + n, f"l{i}.right." + n) for n in right]
     return rules
+
+
+def rifizen_name_rules(cfg) -> List[NameRule]:
+    """Rifizen checkpoints name a layer's tensors ``l<i>.norm1``, ``norm1b``, ``norm2``, ``norm2b`` (the norms before and
+    behind the two branches), ``l<i>.mix.left.{q,k,v,o}`` and ``l<i>.mix.right.{q,k,v,g,o}``, ``mix.left.out`` and
+    ``mix.right.out`` (the norms of the two mixers' results) and ``l<i>.mlp.{up,down}`` (a mixture:
+    ``mlp.e<j>.{gate,up,down}``, ``mlp.router``, ``mlp.router.b``); beside them ``embed``, ``loop.step`` (one vector a
+    pass of the loop), ``final.norm`` and ``head``."""
+    L = "l{}."
+    rules = [
+        NameRule("embed", "embed.weight"),
+        NameRule("loop.step", "loop.step"),
+        NameRule("final.norm", "final_norm.weight"),
+        NameRule("head", "head.weight"),
+        NameRule(L + "mix.left.out", L + "left_out.weight"),
+        NameRule(L + "mix.right.out", L + "right_out.weight"),
+        NameRule(L + "mlp.up", L + "mlp.up.weight"),
+        NameRule(L + "mlp.down", L + "mlp.down.weight"),
+        NameRule(L + "mlp.router", L + "mlp.router.weight"),
+        NameRule(L + "mlp.router.b", L + "mlp.router.bias"),
+        NameRule(L + "mlp.e{}.gate", L + "mlp.experts.{}.w1.weight"),
+        NameRule(L + "mlp.e{}.up", L + "mlp.experts.{}.w3.weight"),
+        NameRule(L + "mlp.e{}.down", L + "mlp.experts.{}.w2.weight"),
+    ]
+    rules += [NameRule(L + n, L + n + ".weight") for n in ("norm1", "norm1b", "norm2", "norm2b")]
+    rules += [NameRule(L + "mix.left." + n, L + f"left.w{n}.weight") for n in ("q", "k", "v", "o")]
+    rules += [NameRule(L + "mix.right." + n, L + "right." + n) for n in ("q", "k", "v", "g", "o")]
+    return rules
