@@ -2,7 +2,7 @@
 bfloat16 weights, synthetic token ids.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 8192] [--layers L]
-                    [--shape 8b|1b|70b] [--workload decode|serve|peaks|small-kernels|attention|products|taluvik|vobolorn|kepevik|nosuzen]
+                    [--shape 8b|1b|70b] [--workload decode|serve|peaks|small-kernels|attention|products|taluvik|vobolorn|kepevik|nosuzen|rifizen]
 
 Everything runs through the generation loop: the scheduler admits the requests, cuts their prompts
 into portions under its token budget, and plans every decode step; the step function runs it; the
@@ -89,8 +89,8 @@ def parse_args(argv=None):
     p.add_argument("--points", default="1,64", help="further decode batch sizes, comma separated ('' for none)")
     p.add_argument("--page-size", type=int, default=16)
     p.add_argument("--shape", default="8b", choices=sorted(SHAPES), help="layer sizes (default: the headline's)")
-    p.add_argument("--workload", default="decode", choices=["decode", "serve", "peaks", "small-kernels", "attention", "products", "taluvik", "vobolorn", "kepevik", "nosuzen"])
-    p.add_argument("--only", default=None, choices=["taluvik", "vobolorn", "kepevik", "nosuzen", "llama"], help="taluvik, vobolorn, kepevik, nosuzen: measure one of the two models only")
+    p.add_argument("--workload", default="decode", choices=["decode", "serve", "peaks", "small-kernels", "attention", "products", "taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen"])
+    p.add_argument("--only", default=None, choices=["taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen", "llama"], help="taluvik, vobolorn, kepevik, nosuzen, rifizen: measure one of the two models only")
     p.add_argument("--token-budget", type=int, default=8192, help="tokens a step may hold (the scheduler cuts prompts to it)")
     p.add_argument("--no-reference-workload", action="store_true",
                    help="leave out the reference's benchmark (2,048-token prompts, 256 new tokens at batch 1, 8, 64)")
@@ -396,6 +396,25 @@ def nosuzen_config(shape: dict, n_layers: int) -> dict:
             "layers": layers}
 
 
+def rifizen_config(shape: dict, n_layers: int) -> dict:
+    """A Rifizen configuration with the layer sizes of ``shape`` (a Llama configuration): the same width, heads and head
+    size in the attention, a window of 4,096; retention with half as many heads, all their channels rotated; the first
+    feed-forward dense with the shape's width inside, the others mixtures of eight experts of a quarter of that width,
+    of which a token uses two.  ``n_layers`` layer runs (at least six): two layers in the middle run twice."""
+    D, H, G, dh, ff = shape["hidden_size"], shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"], shape["intermediate_size"]
+    h2 = max(H // 2, 1)
+    pair = {"left": {"heads": H, "kv_heads": G, "dim": dh, "vdim": dh, "scale": dh ** -0.5, "softcap": 30.0, "mask": {"size": 4096}},
+            "right": {"heads": h2, "dim": dh, "vdim": dh, "decay": [1.0 - 2.0 ** (-5.0 - 7.0 * h / h2) for h in range(h2)],
+                      "rot": {"dims": dh, "base": shape["rope_theta"]}}}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 8, "top": 2}}
+    n = n_layers - 2 if n_layers >= 6 else n_layers
+    d = {"architecture": "Rifizen", "vocab": shape["vocab_size"], "width": D, "norm": {"eps": 1e-6},
+         "layers": [{"type": "parallel", "mixer": pair, "mlp": {"kind": "dense", "ff": ff} if i == 0 else moe} for i in range(n)]}
+    if n < n_layers:
+        d["loop"] = {"start": n // 2, "stop": n // 2 + 2, "times": 2}
+    return d
+
+
 def taluvik_run(args, shape) -> int:
     """Prefill and decode of a Taluvik (or, ``--workload vobolorn``, a Vobolorn) model beside a Llama model of the
     same layer sizes and number of layers, both with random weights, both through the same engine, scheduler and
@@ -411,9 +430,17 @@ def taluvik_run(args, shape) -> int:
     n_layers = args.layers or 8
     batches = [args.batch] + [int(b) for b in args.points.split(",") if b]
     pages_per_req = -(-max(args.context, args.prefill_tokens) // args.page_size) + 1
-    design = {"vobolorn": "Vobolorn", "kepevik": "Kepevik", "nosuzen": "Nosuzen"}.get(args.workload, "Taluvik")
+    design = {"vobolorn": "Vobolorn", "kepevik": "Kepevik", "nosuzen": "Nosuzen", "rifizen": "Rifizen"}.get(args.workload, "Taluvik")
     beside = "Llama"
-    if args.workload == "nosuzen":
+    if args.workload == "rifizen":
+        # beside the design nearest to it: Nosuzen, which has windowed attention beside a linear attention and routed feed-forwards too
+        from torchllms_amd.config.nosuzen import NosuzenConfig
+        from torchllms_amd.config.rifizen import RifizenConfig
+
+        beside = "Nosuzen"
+        configs = {"rifizen": RifizenConfig.from_dict(rifizen_config(shape, n_layers)),
+                   "nosuzen": NosuzenConfig.from_dict(nosuzen_config(shape, n_layers))}
+    elif args.workload == "nosuzen":
         # beside the design nearest to it: Kepevik, whose layers hold attention beside a recurrence and routed feed-forwards too
         from torchllms_amd.config.kepevik import KepevikConfig
         from torchllms_amd.config.nosuzen import NosuzenConfig
@@ -696,7 +723,7 @@ def main(argv=None) -> int:
         return products_run(args, shape)
     if args.workload == "peaks":
         return peaks_run(args)
-    if args.workload in ("taluvik", "vobolorn", "kepevik", "nosuzen"):
+    if args.workload in ("taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen"):
         return taluvik_run(args, shape)
     import torch
 

@@ -530,97 +530,136 @@ __global__ void __launch_bounds__(kSandwichThreads) post_norm_add_norm_kernel(co
   for (int i = threadIdx.x; i < hidden; i += kSandwichThreads) g.rows[r * hidden + i] = from_f32<T>(row_l[i] * inv2 * g.w_next[i]);
 }
 
-// The same for few rows of up to HELD * 256 elements: a launch is then as long as a row's trips to memory, so everything
-// a thread needs is asked for at once (an element past the end is the row's first once more, and not used).  Operation
-// for operation the kernel above: the same bits.
-template <typename T, int HELD, bool PAIR>
-__global__ void __launch_bounds__(kSandwichThreads) post_norm_add_norm_held_kernel(const SandwichArgs<T> g) {
+// Four elements of a row as floats, from memory aligned to them.
+__device__ __forceinline__ void load_four(const float* p, float (&v)[4]) {
+  const float4 x = *reinterpret_cast<const float4*>(p);
+  v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
+}
+__device__ __forceinline__ void store_four(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = float4{v[0], v[1], v[2], v[3]}; }
+struct alignas(8) Bf16Four { bf16_t e[4]; };
+__device__ __forceinline__ void store_four(bf16_t* p, const float (&v)[4]) {
+  *reinterpret_cast<Bf16Four*>(p) = Bf16Four{{from_f32<bf16_t>(v[0]), from_f32<bf16_t>(v[1]), from_f32<bf16_t>(v[2]), from_f32<bf16_t>(v[3])}};
+}
+// ... and as they come from memory, for a later look at them.
+template <typename T> struct RawFour { T e[4]; };
+template <> struct alignas(16) RawFour<float> { float e[4]; };
+template <> struct alignas(8) RawFour<bf16_t> { bf16_t e[4]; };
+
+// The sum over a block of up to 16 waves, in a fixed order.
+__device__ __forceinline__ float sum_of_block(float v, float* scratch) {
+  v = wave_sum(v);
+  __syncthreads();
+  if (threadIdx.x % kWave == 0) scratch[threadIdx.x / kWave] = v;
+  __syncthreads();
+  float total = 0.f;
+  for (int w = 0; w < (int)blockDim.x / kWave; ++w) total += scratch[w];
+  return total;
+}
+
+// The same for rows of a multiple of four elements (up to 4 * CH of them a thread), held in registers: everything a
+// thread needs is asked for at once, four elements a load, so a launch of few rows is one trip to memory long and one
+// of many keeps enough of them in flight.  A row's sums have an order that its width alone decides.
+template <typename T, bool PAIR, int CH, int THREADS>
+__global__ void __launch_bounds__(THREADS) post_norm_add_norm_held_kernel(const SandwichArgs<T> g) {
 #pragma clang fp contract(off)
-  __shared__ float scratch[kSandwichThreads / kWave];
+  __shared__ float scratch[THREADS / kWave];
   const int hidden = g.hidden;
   const size_t r = blockIdx.x;
   const T* yr = g.y + r * hidden;
   float* sr = g.stream + r * hidden;
-  T yraw[HELD], braw[PAIR ? HELD : 1];
-  float sv[HELD], wp[HELD], wn[HELD], av[HELD], wa[PAIR ? HELD : 1], wb[PAIR ? HELD : 1];
+  RawFour<T> yraw[CH], braw[PAIR ? CH : 1];
+  float sv[CH][4], wp[CH][4], wn[CH][4], wa[PAIR ? CH : 1][4], wb[PAIR ? CH : 1][4];
+  int at[CH];
+  bool in[CH];
 #pragma unroll
-  for (int c = 0; c < HELD; ++c) {
-    const int i = threadIdx.x + c * kSandwichThreads;
-    const int at = i < hidden ? i : 0;
-    yraw[c] = yr[at];
-    sv[c] = sr[at];
-    wp[c] = g.w_post[at];
-    wn[c] = g.w_next ? g.w_next[at] : 0.f;
-    av[c] = g.add ? g.add[at] : 0.f;
+  for (int c = 0; c < CH; ++c) {
+    const int i = 4 * ((int)threadIdx.x + c * (int)blockDim.x);
+    in[c] = i < hidden;
+    at[c] = in[c] ? i : 0;  // (elements past the end are the row's first once more, and not used)
+    yraw[c] = *reinterpret_cast<const RawFour<T>*>(yr + at[c]);
+    if constexpr (PAIR) braw[c] = *reinterpret_cast<const RawFour<T>*>(g.b + r * hidden + at[c]);
+    load_four(sr + at[c], sv[c]);
     if constexpr (PAIR) {
-      braw[c] = g.b[r * hidden + at];
-      wa[c] = g.w_a[at];
-      wb[c] = g.w_b[at];
+      load_four(g.w_a + at[c], wa[c]);
+      load_four(g.w_b + at[c], wb[c]);
     }
+    load_four(g.w_post + at[c], wp[c]);
+    load_four((g.w_next ? g.w_next : g.w_post) + at[c], wn[c]);
   }
-  float yv[HELD], bv[PAIR ? HELD : 1];
+  float yv[CH][4], bv[PAIR ? CH : 1][4];
   float ss = 0.f, ss_b = 0.f;
 #pragma unroll
-  for (int c = 0; c < HELD; ++c) {
-    const bool in = threadIdx.x + c * kSandwichThreads < hidden;
-    yv[c] = in ? to_f32(yraw[c]) : 0.f;
-    ss += yv[c] * yv[c];
-    if constexpr (PAIR) {
-      bv[c] = in ? to_f32(braw[c]) : 0.f;
-      ss_b += bv[c] * bv[c];
+  for (int c = 0; c < CH; ++c)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      yv[c][e] = in[c] ? to_f32(yraw[c].e[e]) : 0.f;
+      ss += yv[c][e] * yv[c][e];
+      if constexpr (PAIR) {
+        bv[c][e] = in[c] ? to_f32(braw[c].e[e]) : 0.f;
+        ss_b += bv[c][e] * bv[c][e];
+      }
     }
-  }
-  ss = block_sum<kSandwichThreads / kWave>(ss, scratch);
+  ss = sum_of_block(ss, scratch);
   if constexpr (PAIR) {
-    ss_b = block_sum<kSandwichThreads / kWave>(ss_b, scratch);
+    ss_b = sum_of_block(ss_b, scratch);
     const float inv_a = 1.0f / sqrtf(ss / (float)hidden + g.eps_a), inv_b = 1.0f / sqrtf(ss_b / (float)hidden + g.eps_b);
     ss = 0.f;
 #pragma unroll
-    for (int c = 0; c < HELD; ++c) {  // (an element past the end is zero in both)
-      yv[c] = g.s_a * (yv[c] * inv_a * wa[c]) + g.s_b * (bv[c] * inv_b * wb[c]);
-      ss += yv[c] * yv[c];
-    }
-    ss = block_sum<kSandwichThreads / kWave>(ss, scratch);
+    for (int c = 0; c < CH; ++c)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {  // (an element past the end is zero in both)
+        yv[c][e] = g.s_a * (yv[c][e] * inv_a * wa[c][e]) + g.s_b * (bv[c][e] * inv_b * wb[c][e]);
+        ss += yv[c][e] * yv[c][e];
+      }
+    ss = sum_of_block(ss, scratch);
   }
   const float inv = 1.0f / sqrtf(ss / (float)hidden + g.eps);
   float s2 = 0.f;
 #pragma unroll
-  for (int c = 0; c < HELD; ++c) {
-    const int i = threadIdx.x + c * kSandwichThreads;
-    if (i < hidden) {
-      sv[c] = sv[c] + yv[c] * inv * wp[c];
-      if (g.add) sv[c] = sv[c] + av[c];
-      sr[i] = sv[c];
-      s2 += sv[c] * sv[c];
+  for (int c = 0; c < CH; ++c) {
+    float av[4] = {0.f, 0.f, 0.f, 0.f};
+    if (g.add) load_four(g.add + at[c], av);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      sv[c][e] = sv[c][e] + yv[c][e] * inv * wp[c][e];
+      if (g.add) sv[c][e] = sv[c][e] + av[e];
+      if (in[c]) s2 += sv[c][e] * sv[c][e];
     }
+    if (in[c]) store_four(sr + at[c], sv[c]);
   }
   if (g.w_next == nullptr) return;
-  s2 = block_sum<kSandwichThreads / kWave>(s2, scratch);
+  s2 = sum_of_block(s2, scratch);
   const float inv2 = 1.0f / sqrtf(s2 / (float)hidden + g.eps_next);
 #pragma unroll
-  for (int c = 0; c < HELD; ++c) {
-    const int i = threadIdx.x + c * kSandwichThreads;
-    if (i < hidden) g.rows[r * hidden + i] = from_f32<T>(sv[c] * inv2 * wn[c]);
+  for (int c = 0; c < CH; ++c) {
+    if (!in[c]) continue;
+    float out[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) out[e] = sv[c][e] * inv2 * wn[c][e];
+    store_four(g.rows + r * hidden + at[c], out);
   }
 }
 
 template <typename T, bool PAIR>
 int launch_sandwich(const SandwichArgs<T>& g, int n, hipStream_t stream) {
-  const size_t lds = (size_t)g.hidden * sizeof(float) * (PAIR ? 2 : 1);
-  const bool few = n <= 2 * tl_device_facts().compute_units;
-  if (few && g.hidden <= 4 * kSandwichThreads)
-    post_norm_add_norm_held_kernel<T, 4, PAIR><<<n, kSandwichThreads, 0, stream>>>(g);
-  else if (few && g.hidden <= 16 * kSandwichThreads)
-    post_norm_add_norm_held_kernel<T, 16, PAIR><<<n, kSandwichThreads, 0, stream>>>(g);
-  else {
-    if (lds + 64 > (size_t)tl_device_facts().lds_bytes)
-      return tl_fail(TL_ERR_UNSUPPORTED, "post_norm_add_norm: rows of %d elements do not fit the LDS", g.hidden);
-    if (lds > 48 * 1024) {
-      hipError_t e = hipFuncSetAttribute((const void*)post_norm_add_norm_kernel<T, PAIR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-      if (e != hipSuccess) return tl_fail(TL_ERR_HIP, "post_norm_add_norm: %s", hipGetErrorString(e));
-    }
-    post_norm_add_norm_kernel<T, PAIR><<<n, kSandwichThreads, lds, stream>>>(g);
+  const int fours = g.hidden / 4;
+  const uintptr_t places = (uintptr_t)g.stream | (uintptr_t)g.w_a | (uintptr_t)g.w_b | (uintptr_t)g.w_post | (uintptr_t)g.w_next | (uintptr_t)g.add;
+  const uintptr_t rows = (uintptr_t)g.y | (uintptr_t)g.b | (uintptr_t)g.rows;
+  if (g.hidden % 4 == 0 && fours <= 4096 && places % 16 == 0 && rows % (4 * sizeof(T)) == 0) {
+    if (fours <= 256) post_norm_add_norm_held_kernel<T, PAIR, 1, 256><<<n, (fours + kWave - 1) / kWave * kWave, 0, stream>>>(g);
+    else if (fours <= 512) post_norm_add_norm_held_kernel<T, PAIR, 2, 256><<<n, 256, 0, stream>>>(g);
+    else if (fours <= 1024) post_norm_add_norm_held_kernel<T, PAIR, 4, 256><<<n, 256, 0, stream>>>(g);
+    else post_norm_add_norm_held_kernel<T, PAIR, 4, 1024><<<n, (fours + 4 * kWave - 1) / (4 * kWave) * kWave, 0, stream>>>(g);
+    return tl_check_launch("post_norm_add_norm");
   }
+  const size_t lds = (size_t)g.hidden * sizeof(float) * (PAIR ? 2 : 1);
+  if (lds + 64 > (size_t)tl_device_facts().lds_bytes)
+    return tl_fail(TL_ERR_UNSUPPORTED, "post_norm_add_norm: rows of %d elements do not fit the LDS", g.hidden);
+  if (lds > 48 * 1024) {
+    hipError_t e = hipFuncSetAttribute((const void*)post_norm_add_norm_kernel<T, PAIR>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return tl_fail(TL_ERR_HIP, "post_norm_add_norm: %s", hipGetErrorString(e));
+  }
+  post_norm_add_norm_kernel<T, PAIR><<<n, kSandwichThreads, lds, stream>>>(g);
   return tl_check_launch("post_norm_add_norm");
 }
 

@@ -57,6 +57,9 @@ _CORE_SIGNATURES = {
     "tl_relu_square": [_P, _I64, _I, _P],
     "tl_retention": [_P, _I, _I, _I, _I, _I, _P, _I, _P, _P, _I64, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P],
     "tl_retention_block_columns": [],
+    "tl_retention_chunks": [_P, _I, _I, _I, _I, _I, _P, _I, _P, _P, _I64, _P, _P, _I, _I, _I, _I, _F, _P, _P, _I, _P, _I, _P],
+    "tl_retention_segment": [],
+    "tl_retention_chunk_channels": [],
     "tl_head_prepare": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _I, _F, _P, _I, _I, _I, _P, _F, _I, _P, _I, _P, _P, _P, _P, _I, _I, _P],
     "tl_branch_norm_add": [_P, _P, _P, _P, _I, _I, _F, _I, _P],
     "tl_rmsnorm_columns": [_P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _F, _P],

@@ -139,7 +139,10 @@ from .routed_ops import (  # noqa: F401
 )
 from .retention_ops import (  # noqa: F401
     RETENTION_MAX_KEY_DIM,
+    RETENTION_SEGMENT,
+    RETENTION_SEGMENTS_FROM,
     retention,
+    retention_segments_supported,
 )
 from .stream_ops import (  # noqa: F401
     MAX_STREAMS,

@@ -217,6 +217,7 @@ class ScanSegments:
     def __init__(self, qo_indptr_host, device, length: int = SCAN_SEGMENT):
         import numpy as np
 
+        self.length = length
         bounds = [int(v) for v in qo_indptr_host]
         segs, row_seg = [], [0]
         for lo, hi in zip(bounds[:-1], bounds[1:]):

@@ -370,7 +370,14 @@ class Retention(Mixer):
         qk, v = self.H * self.dk, self.H * self.dv
         rot = self.position.rotary_args()
         table = step_table(rot, ctx) if rot is not None and rot.rotary_dim > 0 else None
+        rotary_dim = rot.rotary_dim if table is not None else 0
         proj = ops.linear(ops.resolved(x), self.w_all)
-        y = ops.retention(proj, 0, qk, 2 * qk, 2 * qk + v, table, rot.rotary_dim if table is not None else 0, self.decay, self.norm_eps,
-                          cache.tensor, 0, ctx.qo_indptr, ctx.slot_ids, self.H, self.dk, self.dv)
+        # of a bfloat16 step with prompts the prompts' rows (behind those of single tokens) run in segments side by side
+        host, segments = ctx.host, None
+        if host.max_q_len >= ops.RETENTION_SEGMENTS_FROM and ops.retention_segments_supported(proj.dtype, self.dk, self.dv, rotary_dim):
+            segments = ctx.scratch.get("retention_segments")
+            if segments is None:
+                segments = ctx.scratch["retention_segments"] = ops.ScanSegments(host.qo_indptr[host.n_decode :], proj.device, ops.RETENTION_SEGMENT)
+        y = ops.retention(proj, 0, qk, 2 * qk, 2 * qk + v, table, rotary_dim, self.decay, self.norm_eps, cache.tensor, 0, ctx.qo_indptr,
+                          ctx.slot_ids, self.H, self.dk, self.dv, segments=segments, single_rows=host.n_decode)
         return ops.linear_to_sum(y, self.w_o)
