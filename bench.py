@@ -28,6 +28,8 @@ a read of 4 GiB with 16-byte loads, a device copy, a loop of MFMA instructions o
 library's large matrix product.  ``--workload small-kernels`` times what a norm kernel adds to a
 replayed graph of large products, without a profiler (under rocprofv3 no dispatch is shorter than
 about 4.6 us, an empty kernel included, so a kernel trace overstates the small kernels of a step).
+``--workload rifizen``: prefill and decode of a Rifizen model (windowed attention with a bias by distance beside retention,
+dense and routed feed-forwards, two layers that run twice) beside a Nosuzen model of the same layer sizes.
 ``--workload nosuzen``: prefill and decode of a Nosuzen model (several residual streams, differential attention behind short
 convolutions with kept first keys, attention through a latent, attention beside gated linear attention, routed
 feed-forwards with grouped routers) beside a Kepevik model of the same layer sizes.

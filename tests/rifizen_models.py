@@ -2,9 +2,9 @@
 
 The configurations differ from each other in every size and constant, and in what a single model may happen to make
 equal or one: heads and kv heads (one of each among them), sizes of keys and values on both sides, rotated channels
-(all, some, none), windows (a single position among them), caps, decays up to 1 (a head that forgets at once is its token's value times the
-sign of q . k but for the norm's eps: rounding shows there, so such heads are tested alone), dense, routed and no feed-forward,
-one choice, several and all, a loop from the first layer, to the last, over one layer, of one pass, and none."""
+(all, some, none), windows (a single position among them), caps, decays up to 1 (a head that forgets at once is its
+token's value times the sign of q . k but for the norm's eps: rounding shows there, so such heads are tested alone),
+dense, routed and no feed-forward, one choice, several and all, a loop from the first layer, to the last, and none."""
 
 from __future__ import annotations
 

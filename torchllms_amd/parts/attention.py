@@ -131,7 +131,7 @@ class Attention(Mixer):
         self.k_norm: Optional[torch.Tensor] = None
         self.vmix: Optional[torch.Tensor] = None
         if qkv_bias and self.extended and not self.prepared:
-            raise ValueError("attention: q/k/v biases together with a unit norm, capped scores, chunks, sinks or values of their own size are not built")
+            raise ValueError("attention: q/k/v biases together with a unit norm, capped scores, chunks, sinks, a bias by distance or values of their own size are not built")
         self.sinks: Optional[torch.Tensor] = None
         self.position = POSITIONS.build(position)
         self.wqkv: Optional[torch.Tensor] = None
@@ -273,9 +273,9 @@ class Attention(Mixer):
         return ops.linear_to_sum(attn, self.wo, may_wait=True)
 
     def _forward_extended(self, x, ctx, cache, n_kv_in_row, rot, table, store):
-        """The layer with a unit norm on queries and keys, capped scores, chunks, sinks or values of their
-        own head size: the projection, then rotation, norm and cache write in one kernel, then the plain
-        attention kernel, which takes all of these."""
+        """The layer with a unit norm on queries and keys, capped scores, chunks, sinks, a bias by distance or values
+        of their own head size: the projection, then rotation, norm and cache write in one kernel, then the
+        attention kernel that takes the sizes."""
         g = cache.group
         qkv = ops.linear(ops.resolved(x), self.wqkv)
         ops.rope_norm_kv_write(

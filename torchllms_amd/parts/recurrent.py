@@ -1,5 +1,6 @@
 """Mixers that carry a state of fixed size per request instead of keys and values: the selective scan
-of a diagonal state-space layer and the gated delta rule, both behind a short causal convolution.
+of a diagonal state-space layer and the gated delta rule, both behind a short causal convolution, the matrix
+memory, gated linear attention and retention.
 
 Everything such a mixer keeps for a request lies in one 32-bit row of its ``StateView`` (the
 convolution's history first, then the recurrence's state); rows are zeroed when a request is admitted,
