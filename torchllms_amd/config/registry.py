@@ -21,6 +21,7 @@ from .vobolorn import ARCHITECTURE as VOBOLORN, VobolornConfig, vobolorn_model_s
 from .kepevik import ARCHITECTURE as KEPEVIK, KepevikConfig, kepevik_model_spec, kepevik_sizes_from_tensors
 from .nosuzen import ARCHITECTURE as NOSUZEN, NosuzenConfig, nosuzen_model_spec, nosuzen_sizes_from_tensors
 from .rifizen import ARCHITECTURE as RIFIZEN, RifizenConfig, rifizen_model_spec
+from .mesolix import ARCHITECTURE as MESOLIX, MesolixConfig, mesolix_model_spec, mesolix_sizes_from_tensors
 
 
 @dataclass(frozen=True)
@@ -272,5 +273,29 @@ register_architecture(
         weight_rules=_rifizen_rules,
         stop_token_ids=_rifizen_stop_ids,
         config_type=RifizenConfig,
+    )
+)
+
+
+def _mesolix_rules(cfg: MesolixConfig):
+    from ..weights.names import mesolix_name_rules
+
+    return mesolix_name_rules(cfg)
+
+
+def _mesolix_stop_ids(cfg: MesolixConfig):
+    eos = cfg.eos_token_id
+    return [] if eos is None else (list(eos) if isinstance(eos, (list, tuple)) else [eos])
+
+
+register_architecture(
+    ArchSpec(
+        name=MESOLIX,
+        config_from_dict=MesolixConfig.from_dict,
+        model_spec=mesolix_model_spec,
+        weight_rules=_mesolix_rules,
+        stop_token_ids=_mesolix_stop_ids,
+        config_type=MesolixConfig,
+        sizes_from_tensors=mesolix_sizes_from_tensors,
     )
 )

@@ -88,6 +88,9 @@ struct DecodeArgs {
   float two_scale_over_cap_log2e;  // ... and this 2 * scale / cap * log2(e): tanh(x) = 1 - 2 / (exp2(2 x log2(e)) + 1)
   const float* sinks;  // per query head, or null: exp(sink) joins the softmax's denominator
   const float* slopes; // per query head, or null: what a capped score loses for every position between key and query
+  const float* dist;   // [query heads][dist_len], or null: what a capped score gains by distance (past the end: the last entry)
+  int dist_len;
+  int n_k_heads;       // heads of the key pages: key head g reads page head g % n_k_heads
   int split_size;     // keys per split, a multiple of 64
   int n_splits;
   float* ws_o;   // [token][q head][split][DH]
@@ -134,8 +137,9 @@ __device__ __forceinline__ void load_value_words(const bf16_t* src, uint32_t* ds
 // kPow2Pages: the page size is a power of two, so a key's page and offset are a shift and a mask;
 // the general kernel divides, inlined at each of the 25 places that look a page up (6.6 KB of code
 // against 4.7).  Both run at the same speed; they are two kernels so that neither carries the
-// other's code and branches.
-template <bool kPow2Pages>
+// other's code and branches.  kDist: the kernel reads a table of what scores gain by distance; its entries are asked for
+// a tile ahead, as everything else.
+template <bool kPow2Pages, bool kDist>
 __global__ void __launch_bounds__(kWaves* kWave, TL_DECODE_MIN_WAVES) attn_decode_kernel(DecodeArgs a) {
   extern __shared__ float red_o[];  // [kWaves][group][DH]: per-wave partial outputs for the block merge
   __shared__ float red_m[kWaves][16], red_l[kWaves][16];
@@ -200,8 +204,21 @@ __global__ void __launch_bounds__(kWaves* kWave, TL_DECODE_MIN_WAVES) attn_decod
   };
   auto block_of = [&](int key) { return kPow2Pages ? key >> a.page_shift : key / a.page_size; };
   auto offset_of = [&](int key) { return kPow2Pages ? key & (a.page_size - 1) : key % a.page_size; };
+  const int kh = kvh % a.n_k_heads;
   auto row_ptr = [&](const bf16_t* pages, int page, int key) {
-    return pages + ((size_t)page * a.n_kv_heads + kvh) * head_elems + (size_t)offset_of(key) * DH;
+    return pages + ((size_t)page * a.n_k_heads + kh) * head_elems + (size_t)offset_of(key) * DH;
+  };
+  const float* dist_row = kDist ? a.dist + (size_t)(kvh * R + (n16 < R ? n16 : 0)) * a.dist_len : nullptr;
+  float gain[4];
+  auto load_gain = [&](int base) {
+    if constexpr (kDist) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int count = base + 4 * g4 + i;
+        const int n = p - (count < keep_al ? count : lo_al + (count - keep_al));
+        gain[i] = dist_row[max(min(n, a.dist_len - 1), 0)];
+      }
+    }
   };
   const int vh = kvh % a.n_v_heads;
   auto value_ptr = [&](int page, int key) {
@@ -253,6 +270,7 @@ __global__ void __launch_bounds__(kWaves* kWave, TL_DECODE_MIN_WAVES) attn_decod
     const TilePages pages_now = fetch_pages(base);
     load_k(base, pages_now);
     load_v(base, pages_now);
+    load_gain(base);
     keep_loads_here();
   }
   for (; base <= split_end; base += kWaves * kTile) {
@@ -277,9 +295,14 @@ __global__ void __launch_bounds__(kWaves* kWave, TL_DECODE_MIN_WAVES) attn_decod
       float sc = c[i] * a.scale_log2e;
       if (a.cap_log2e > 0.f)  // (the same in every lane)
         sc = a.cap_log2e * (1.0f - 2.0f * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(c[i] * a.two_scale_over_cap_log2e) + 1.0f));
-      sc = fmaf(-slope_log2e, (float)(p - (count < keep_al ? count : key)), sc);
+      if constexpr (kDist) sc = fmaf(gain[i], 1.4426950408889634f, sc);
+      else sc = fmaf(-slope_log2e, (float)(p - (count < keep_al ? count : key)), sc);
       s[i] = valid ? sc : -INFINITY;
       tmax = fmaxf(tmax, s[i]);
+    }
+    if constexpr (kDist) {
+      load_gain(next);
+      keep_loads_here();
     }
     tmax = fmaxf(tmax, __shfl_xor(tmax, 16, kWave));
     tmax = fmaxf(tmax, __shfl_xor(tmax, 32, kWave));
@@ -427,19 +450,23 @@ TL_EXPORT int tl_attn_decode_head_dim() { return DH; }
 // null) join the denominators, slopes (likewise) are taken off the capped scores for every position of distance.  Every token is one query at positions[t] of request row token_seq[t].  split_size: keys per
 // split (a multiple of 64); n_splits >= ceil(longest visible range / split_size), counted from the
 // 16-aligned first visible key, plus the kept first keys rounded up to 16.  keep_first, n_v_heads (0: n_kv_heads),
-// v_pitch / v_offset and out_pitch / out_offset (0: DH): see DecodeArgs.  ws_o / ws_ml: workspaces (unused when n_splits == 1).
+// v_pitch / v_offset, out_pitch / out_offset (0: DH), dist / dist_len and n_k_heads (0: n_kv_heads): see DecodeArgs.  ws_o / ws_ml: workspaces (unused when n_splits == 1).
 TL_EXPORT int tl_attn_decode(const void* q, int q_stride, void* out, int out_stride, const void* k_pages,
                              const void* v_pages, const int32_t* token_seq, const int32_t* positions,
                              const int32_t* block_table, int bt_stride, int n_tokens, int n_q_heads,
                              int n_kv_heads, int head_dim, int page_size, int window, float scale,
                              int split_size, int n_splits, float* ws_o, float* ws_ml, float softcap, int chunk,
                              const float* sinks, int keep_first, int n_v_heads, int v_pitch, int v_offset, int out_pitch,
-                             int out_offset, const float* slopes, hipStream_t stream) {
+                             int out_offset, const float* slopes, const float* dist, int dist_len, int n_k_heads,
+                             hipStream_t stream) {
   if (head_dim != DH) return variant_fail(TL_ERR_ARG, "attn_decode: built for head_dim %d, called with %d", DH, head_dim);
   if (n_tokens < 0 || n_q_heads <= 0 || n_kv_heads <= 0 || page_size <= 0 || bt_stride <= 0 || window < 0 || chunk < 0 || softcap < 0)
     return variant_fail(TL_ERR_ARG, "attn_decode: bad sizes");
   if (n_q_heads % n_kv_heads) return variant_fail(TL_ERR_ARG, "attn_decode: %d query heads are not a multiple of %d kv heads", n_q_heads, n_kv_heads);
   if (n_v_heads <= 0) n_v_heads = n_kv_heads;
+  if (n_k_heads <= 0) n_k_heads = n_kv_heads;
+  if (n_kv_heads % n_k_heads || (dist && (dist_len <= 0 || slopes)))
+    return variant_fail(TL_ERR_ARG, "attn_decode: heads of the key pages, or a table by distance, that do not fit");
   if (v_pitch <= 0) v_pitch = DH;
   if (out_pitch <= 0) out_pitch = DH;
   if (keep_first < 0 || n_kv_heads % n_v_heads || v_offset < 0 || v_offset + DH > v_pitch || out_offset < 0 || out_offset + DH > out_pitch
@@ -462,7 +489,7 @@ TL_EXPORT int tl_attn_decode(const void* q, int q_stride, void* out, int out_str
   for (int sh = 0; sh < 31; ++sh)
     if ((1 << sh) == page_size) a.page_shift = sh;
   a.scale_log2e = scale * 1.4426950408889634f;
-  a.chunk = chunk; a.sinks = sinks; a.slopes = slopes;
+  a.chunk = chunk; a.sinks = sinks; a.slopes = slopes; a.dist = dist; a.dist_len = dist_len; a.n_k_heads = n_k_heads;
   a.keep_first = keep_first; a.n_v_heads = n_v_heads; a.v_pitch = v_pitch; a.v_offset = v_offset;
   a.out_pitch = out_pitch; a.out_offset = out_offset;
   a.cap_log2e = softcap > 0 ? softcap * 1.4426950408889634f : 0.f;
@@ -471,10 +498,14 @@ TL_EXPORT int tl_attn_decode(const void* q, int q_stride, void* out, int out_str
   dim3 grid(n_splits, n_kv_heads, n_tokens);
   const int threads = kWaves * kWave;
   const size_t lds = (size_t)kWaves * R * DH * sizeof(float);
-  if (a.page_shift >= 0)
-    attn_decode_kernel<true><<<grid, threads, lds, stream>>>(a);
+  if (a.page_shift >= 0 && dist)
+    attn_decode_kernel<true, true><<<grid, threads, lds, stream>>>(a);
+  else if (a.page_shift >= 0)
+    attn_decode_kernel<true, false><<<grid, threads, lds, stream>>>(a);
+  else if (dist)
+    attn_decode_kernel<false, true><<<grid, threads, lds, stream>>>(a);
   else
-    attn_decode_kernel<false><<<grid, threads, lds, stream>>>(a);
+    attn_decode_kernel<false, false><<<grid, threads, lds, stream>>>(a);
   hipError_t e = hipGetLastError();
   if (e != hipSuccess) return variant_fail(TL_ERR_HIP, "attn_decode: %s", hipGetErrorString(e));
   if (n_splits > 1) {

@@ -10,7 +10,8 @@
 // visible behind a window (keep_first: a query also sees the positions below it that lie before its window), and
 // values with fewer heads than the keys (key head g reads value head g mod n_v_heads: several score maps over
 // the same values), and a bias by distance (slopes: a number per query head that is taken off the capped score for
-// every position between key and query).
+// every position between key and query; or dist: a table [query heads][dist_len] of what is added to the capped score
+// by distance, distances past its end taking its last entry).
 #include <limits.h>
 
 #include "common.h"
@@ -62,7 +63,15 @@ struct Query {
   float scale, softcap;
   int pos;                  // the query's position, and what a position of distance costs its head
   float slope;
+  const float* dist;        // or (not null) what its head's score gains by distance, dist_len entries
+  int dist_len;
 };
+
+// What the bias by distance makes of a capped score at distance n.
+__device__ __forceinline__ float biased(float s, int n, float slope, const float* dist, int dist_len) {
+#pragma clang fp contract(off)
+  return dist ? s + dist[min(n, dist_len - 1)] : s - slope * (float)n;
+}
 
 // The first position a query at position p sees: behind a window of `window` keys (0: none) and inside
 // its own chunk of `chunk` positions (0: none).
@@ -124,7 +133,7 @@ __device__ __forceinline__ void block_partial(const Query<T>& a, int j0, int lan
     } else {
       for (int d = 0; d < a.head_dim; ++d) dot = fmaf(a.qs[d], to_f32(kr[d]), dot);
     }
-    s = capped(dot * a.scale, a.softcap) - a.slope * (float)(a.pos - j);
+    s = biased(capped(dot * a.scale, a.softcap), a.pos - j, a.slope, a.dist, a.dist_len);
   }
   m_b = wave_max(s);
   const float pj = valid ? expf(s - m_b) : 0.f;
@@ -182,7 +191,7 @@ __device__ __forceinline__ Query<T> make_query(const float* qs, const T* k_pages
                                                const int32_t* block_table, int bt_stride, int t, int h, int n_q_heads,
                                                int n_kv_heads, int head_dim, int page_size, int window, float scale,
                                                float softcap, int chunk, int v_dim, int v_pitch, int keep_first,
-                                               int n_v_heads, const float* slopes) {
+                                               int n_v_heads, const float* slopes, const float* dist, int dist_len) {
   Query<T> a;
   a.qs = qs; a.k_pages = k_pages; a.v_pages = v_pages;
   a.bt = block_table + (size_t)token_seq[t] * bt_stride;
@@ -195,6 +204,8 @@ __device__ __forceinline__ Query<T> make_query(const float* qs, const T* k_pages
   a.scale = scale; a.softcap = softcap;
   a.pos = a.p;
   a.slope = slopes ? slopes[h] : 0.f;
+  a.dist = dist ? dist + (size_t)h * dist_len : nullptr;
+  a.dist_len = dist_len;
   return a;
 }
 
@@ -229,7 +240,7 @@ attention_generic_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ 
                          const int32_t* __restrict__ block_table, int bt_stride, int n_q_heads,
                          int n_kv_heads, int head_dim, int page_size, int window, float scale, float softcap,
                          int chunk, const float* __restrict__ sinks, int v_dim, int v_pitch, int keep_first, int n_v_heads,
-                         const float* __restrict__ slopes) {
+                         const float* __restrict__ slopes, const float* __restrict__ dist, int dist_len) {
   __shared__ float q_lds[kWavesPerBlock][kMaxKeyDim];
   const int t = blockIdx.x;
   const int wave = threadIdx.x / kWave;
@@ -242,7 +253,7 @@ attention_generic_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ 
   __syncthreads();
   const Query<T> a = make_query<T>(q_lds[wave], k_pages, v_pages, token_seq, positions, block_table, bt_stride, t, h,
                                    n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, v_dim, v_pitch, keep_first, n_v_heads,
-                                   slopes);
+                                   slopes, dist, dist_len);
   float acc[kChanPerLane];
 #pragma unroll
   for (int c = 0; c < kChanPerLane; ++c) acc[c] = 0.f;
@@ -272,7 +283,7 @@ constexpr int kTilePad = 4;  // floats between LDS rows beyond head_dim: rows st
 template <bool VEC, int CH>
 __device__ __forceinline__ void block_partial_lds(const float* qs, const float* k_t, const float* v_t, int pitch,
                                                   int pitch_v, int head_dim, int v_dim, int lo, int p, float scale,
-                                                  float softcap, float slope, int pos, int j0, int lane,
+                                                  float softcap, float slope, const float* dist, int dist_len, int pos, int j0, int lane,
                                                   float& m_b, float& l_b, float (&o_b)[kChanPerLane]) {
 #pragma clang fp contract(off)
   const int j = j0 + lane;
@@ -291,7 +302,7 @@ __device__ __forceinline__ void block_partial_lds(const float* qs, const float* 
     } else {
       for (int d = 0; d < head_dim; ++d) dot = fmaf(qs[d], kr[d], dot);
     }
-    s = capped(dot * scale, softcap) - slope * (float)(pos - j);
+    s = biased(capped(dot * scale, softcap), pos - j, slope, dist, dist_len);
   }
   m_b = wave_max(s);
   const float pj = valid ? expf(s - m_b) : 0.f;
@@ -337,7 +348,7 @@ attention_tile_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ out
                       const int32_t* __restrict__ block_table, int bt_stride, int n_tokens, int n_q_heads,
                       int n_kv_heads, int head_dim, int page_size, int window, float scale, int heads_per_block,
                       float softcap, int chunk, const float* __restrict__ sinks, int v_dim, int v_pitch, int keep_first,
-                      int n_v_heads, const float* __restrict__ slopes) {
+                      int n_v_heads, const float* __restrict__ slopes, const float* __restrict__ dist, int dist_len) {
   extern __shared__ __attribute__((aligned(16))) float tile_lds[];
   const int pitch = head_dim + kTilePad, pitch_v = v_dim + kTilePad;
   float* q_lds = tile_lds;                          // [kTileWaves][head_dim]
@@ -357,7 +368,7 @@ attention_tile_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ out
   for (int d = lane; d < head_dim; d += kWave) q_lds[wave * head_dim + d] = to_f32(qv[d]);
   const Query<T> a = make_query<T>(q_lds + wave * head_dim, k_pages, v_pages, token_seq, positions, block_table,
                                    bt_stride, t, h, n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap,
-                                   chunk, v_dim, v_pitch, keep_first, n_v_heads, slopes);
+                                   chunk, v_dim, v_pitch, keep_first, n_v_heads, slopes, dist, dist_len);
   // what the whole block sees: the same for every thread, from the tokens' own entries
   const int last = min(t0 + QT, n_tokens) - 1;
   const int seq0 = token_seq[t0];
@@ -418,7 +429,7 @@ attention_tile_kernel(const T* __restrict__ q, int q_stride, T* __restrict__ out
       __syncthreads();
       if (p_w >= lo_w && j0 >= lo_w - lo_w % kWave && j0 <= p_w) {  // (uniform per wave)
         float m_b, l_b, o_b[kChanPerLane];
-        block_partial_lds<VEC, CH>(a.qs, k_t, v_t, pitch, pitch_v, head_dim, v_dim, lo_w, p_w, scale, softcap, a.slope, a.pos, j0, lane,
+        block_partial_lds<VEC, CH>(a.qs, k_t, v_t, pitch, pitch_v, head_dim, v_dim, lo_w, p_w, scale, softcap, a.slope, a.dist, a.dist_len, a.pos, j0, lane,
                                    m_b, l_b, o_b);
         merge_block(m, l, acc, m_b, l_b, o_b);
       }
@@ -450,7 +461,7 @@ attention_blocks_kernel(const T* __restrict__ q, int q_stride, const T* __restri
                         const int32_t* __restrict__ positions, const int32_t* __restrict__ block_table, int bt_stride,
                         int n_q_heads, int n_kv_heads, int head_dim, int page_size, int window, float scale,
                         float* __restrict__ partials, int max_blocks, float softcap, int chunk, int v_dim, int v_pitch,
-                        int keep_first, int n_v_heads, const float* __restrict__ slopes) {
+                        int keep_first, int n_v_heads, const float* __restrict__ slopes, const float* __restrict__ dist, int dist_len) {
   __shared__ float q_lds[kWavesPerBlock][kMaxKeyDim];
   const int t = blockIdx.x;
   const int r = blockIdx.z;
@@ -464,7 +475,7 @@ attention_blocks_kernel(const T* __restrict__ q, int q_stride, const T* __restri
   __syncthreads();
   const Query<T> a = make_query<T>(q_lds[wave], k_pages, v_pages, token_seq, positions, block_table, bt_stride, t, h,
                                    n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, v_dim, v_pitch, keep_first, n_v_heads,
-                                   slopes);
+                                   slopes, dist, dist_len);
   // the blocks of the kept first keys come first, then those of positions lo .. p
   const int kept_blocks = (a.keep + kWave - 1) / kWave;
   Query<T> b = a;
@@ -542,14 +553,15 @@ attention_join_kernel(T* __restrict__ out, int out_stride, const int32_t* __rest
 // q: element (t, h, d) at q + t*q_stride + h*head_dim + d.  out likewise with out_stride.
 // pages: [page][n_kv_heads][page_size][head_dim].  token_seq[t]: row of block_table;
 // positions[t]: absolute position; the token sees positions max(0, p-window+1)..p (window 0: all).  slopes: one float
-// per query head (or null) that a capped score loses for every position between its key and the query.
+// per query head (or null) that a capped score loses for every position between its key and the query; dist: a table
+// [n_q_heads][dist_len] (or null) of what it gains by distance instead.
 TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int out_stride,
                                    const void* k_pages, const void* v_pages, const int32_t* token_seq,
                                    const int32_t* positions, const int32_t* block_table, int bt_stride,
                                    int n_tokens, int n_q_heads, int n_kv_heads, int head_dim,
                                    int page_size, int window, float scale, float softcap, int chunk,
                                    const float* sinks, int v_dim, int v_pitch, int dtype, int keep_first, int n_v_heads,
-                                   const float* slopes, hipStream_t stream) {
+                                   const float* slopes, const float* dist, int dist_len, hipStream_t stream) {
   TL_REQUIRE(n_tokens >= 0 && n_q_heads > 0 && n_kv_heads > 0 && page_size > 0 && bt_stride > 0,
              "attention: bad sizes");
   TL_REQUIRE(n_q_heads % n_kv_heads == 0, "attention: %d query heads are not a multiple of %d kv heads",
@@ -564,6 +576,7 @@ TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int o
   TL_REQUIRE(n_kv_heads % n_v_heads == 0, "attention: %d key heads are not a multiple of %d value heads", n_kv_heads, n_v_heads);
   if (v_dim <= 0 || v_dim > kMaxHeadDim)
     return tl_fail(TL_ERR_UNSUPPORTED, "attention: values of head size %d outside 1..%d", v_dim, kMaxHeadDim);
+  TL_REQUIRE(dist == nullptr || (dist_len > 0 && slopes == nullptr), "attention: a table by distance needs entries, and takes the place of slopes");
   if (n_tokens == 0) return TL_OK;
   dim3 grid(n_tokens, (n_q_heads + kWavesPerBlock - 1) / kWavesPerBlock);
   // rows of the pages start at multiples of head_dim elements from an allocation's start
@@ -586,7 +599,7 @@ TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int o
     attention_tile_kernel<T, VEC, CH><<<tgrid, kTileWaves * kWave, lds, stream>>>(                               \
         (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pages, (const T*)v_pages, token_seq, positions,  \
         block_table, bt_stride, n_tokens, n_q_heads, n_kv_heads, head_dim, page_size, window, scale, hb, softcap, \
-        chunk, sinks, v_dim, v_pitch, keep_first, n_v_heads, slopes);                                            \
+        chunk, sinks, v_dim, v_pitch, keep_first, n_v_heads, slopes, dist, dist_len);                            \
   } while (0)
 #define TL_TILE_LAUNCH(T, VEC)                                                                                   \
   do {                                                                                                           \
@@ -612,7 +625,7 @@ TL_EXPORT int tl_attention_generic(const void* q, int q_stride, void* out, int o
   attention_generic_kernel<T, VEC><<<grid, kWavesPerBlock * kWave, 0, stream>>>(                            \
       (const T*)q, q_stride, (T*)out, out_stride, (const T*)k_pages, (const T*)v_pages, token_seq, positions, \
       block_table, bt_stride, n_q_heads, n_kv_heads, head_dim, page_size, window, scale, softcap, chunk, sinks, v_dim, v_pitch, \
-      keep_first, n_v_heads, slopes)
+      keep_first, n_v_heads, slopes, dist, dist_len)
   if (dtype == TL_F32) {
     if (vec) TL_ATTN_LAUNCH(float, true);
     else TL_ATTN_LAUNCH(float, false);
@@ -636,8 +649,8 @@ TL_EXPORT int tl_attention_generic_split(const void* q, int q_stride, void* out,
                                          int n_tokens, int n_q_heads, int n_kv_heads, int head_dim,
                                          int page_size, int window, float scale, float softcap, int chunk,
                                          const float* sinks, int v_dim, int v_pitch, int dtype, int max_blocks,
-                                         float* partials, int keep_first, int n_v_heads, const float* slopes,
-                                         hipStream_t stream) {
+                                         float* partials, int keep_first, int n_v_heads, const float* slopes, const float* dist,
+                                         int dist_len, hipStream_t stream) {
   TL_REQUIRE(n_tokens >= 0 && n_q_heads > 0 && n_kv_heads > 0 && page_size > 0 && bt_stride > 0,
              "attention: bad sizes");
   TL_REQUIRE(n_q_heads % n_kv_heads == 0, "attention: %d query heads are not a multiple of %d kv heads",
@@ -654,6 +667,7 @@ TL_EXPORT int tl_attention_generic_split(const void* q, int q_stride, void* out,
     return tl_fail(TL_ERR_UNSUPPORTED, "attention: values of head size %d outside 1..%d", v_dim, kMaxHeadDim);
   TL_REQUIRE(max_blocks >= 1 && max_blocks <= 65535 && partials != nullptr, "attention: max_blocks=%d outside 1..65535, or no workspace", max_blocks);
   TL_REQUIRE(n_tokens <= 65535, "attention: the split form takes at most 65535 tokens");
+  TL_REQUIRE(dist == nullptr || (dist_len > 0 && slopes == nullptr), "attention: a table by distance needs entries, and takes the place of slopes");
   if (n_tokens == 0) return TL_OK;
   const int head_blocks = (n_q_heads + kWavesPerBlock - 1) / kWavesPerBlock;
   dim3 grid(n_tokens, head_blocks, max_blocks);
@@ -664,7 +678,7 @@ TL_EXPORT int tl_attention_generic_split(const void* q, int q_stride, void* out,
     attention_blocks_kernel<T, VEC><<<grid, kWavesPerBlock * kWave, 0, stream>>>(                               \
         (const T*)q, q_stride, (const T*)k_pages, (const T*)v_pages, token_seq, positions, block_table, bt_stride, \
         n_q_heads, n_kv_heads, head_dim, page_size, window, scale, partials, max_blocks, softcap, chunk, v_dim, v_pitch,  \
-        keep_first, n_v_heads, slopes);                                                                         \
+        keep_first, n_v_heads, slopes, dist, dist_len);                                                         \
     int rc = tl_check_launch("attention_blocks");                                                               \
     if (rc != TL_OK) return rc;                                                                                 \
     attention_join_kernel<T><<<grid_join, kWavesPerBlock * kWave, 0, stream>>>(                                 \

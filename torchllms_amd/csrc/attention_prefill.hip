@@ -111,6 +111,10 @@ struct PrefillArgs {
   const float* sinks;               // per query head, or null: exp(sink) joins the softmax's denominator
   const float* slopes;              // per query head, or null: what a capped score loses for every position between key and query
   float inv_scale;                  // 1 / softmax scale: the pipeline's scores are raw products
+  const float* dist;                // [query heads][dist_len], or null: what a score gains by distance (past the end: the last entry)
+  int dist_len;
+  int dist_pitch;                   // > 0: a block's heads of that table lie in its LDS, so many entries apart
+  int n_k_heads;                    // heads of the key pages: key head g reads page head g % n_k_heads
 };
 
 typedef unsigned int u32x2_t __attribute__((ext_vector_type(2)));
@@ -168,10 +172,11 @@ __device__ __forceinline__ u32x2_t lds_transposed(const bf16_t* src) {
 // needs whose blocks all fit the GPU at once and whose time is therefore that of its longest block.
 // MODE 0: no lower bound and no cap; 1: a lower bound (a window, chunks, or both); 2: a lower bound and capped scores;
 // 3: a lower bound, and before it the first keep_first positions, which come as tiles of their own ahead of the others;
-// 4: a lower bound and a bias by distance; 5: a lower bound, capped scores and a bias by distance.
+// 4: a lower bound and a bias by distance; 5: a lower bound, capped scores and a bias by distance; 6: a lower bound and a
+// table of what scores gain by distance.
 template <int RP, int MODE, int GROUPS>
 __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) attn_prefill_kernel(PrefillArgs a) {
-  constexpr bool WINDOWED = MODE >= 1, CAPPED = MODE == 2 || MODE == 5, KEPT = MODE == 3, BIASED = MODE >= 4;
+  constexpr bool WINDOWED = MODE >= 1, CAPPED = MODE == 2 || MODE == 5, KEPT = MODE == 3, BIASED = MODE == 4 || MODE == 5, TABLE = MODE == 6;
   constexpr int QB = kCols / RP;  // queries per block
 
   const int tile = blockIdx.y;  // the host lists the tiles in the order that balances the launch
@@ -231,6 +236,22 @@ __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) 
       if (!col_ok[i]) qreg[i][u].u = u32x4_t{0u, 0u, 0u, 0u};
     }
   }
+  // (TABLE) in units of the raw products: where the lane's columns read the table, and its last entries
+  extern __shared__ __attribute__((aligned(16))) float dist_l[];
+  int col_row[NC];
+  float col_far[NC];
+  if constexpr (TABLE) {
+#pragma unroll
+    for (int i = 0; i < NC; ++i) {
+      col_far[i] = a.dist[(size_t)col_head[i] * a.dist_len + a.dist_len - 1] * a.inv_scale;
+      col_row[i] = a.dist_pitch > 0 ? (col_head[i] - kvh * R) * a.dist_pitch : col_head[i] * a.dist_len;
+    }
+    if (a.dist_pitch > 0)  // (read behind the barrier before the first scores)
+      for (int e = threadIdx.x; e < R * a.dist_pitch; e += GROUPS * kWaves * kWave) {
+        const int hh = e / a.dist_pitch, n = min(e % a.dist_pitch, a.dist_len - 1);
+        dist_l[e] = a.dist[(size_t)(kvh * R + hh) * a.dist_len + n] * a.inv_scale;
+      }
+  }
   float m_run[NC];
   float4_t acc[NC][DT];
 #pragma unroll
@@ -251,8 +272,8 @@ __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) 
   // that may be read, and their scores are masked.  Addresses are a page's offset (one 64-bit
   // multiply-add per load) plus what does not depend on the page.
   const int blk_lo = key_lo >> a.page_shift, blk_hi = key_hi >> a.page_shift;
-  const unsigned page_bytes = (unsigned)a.n_kv_heads * (unsigned)a.page_size * DH * 2;  // all kv heads of a page
-  const char* const k_head = reinterpret_cast<const char*>(a.k_pages) + (size_t)kvh * head_elems * 2;  // this kv head's rows in page 0
+  const unsigned page_bytes = (unsigned)a.n_k_heads * (unsigned)a.page_size * DH * 2;  // all key heads of a page
+  const char* const k_head = reinterpret_cast<const char*>(a.k_pages) + (size_t)(kvh % a.n_k_heads) * head_elems * 2;  // this head's rows in page 0
   const unsigned v_row_bytes = (unsigned)a.v_pitch * 2;
   const unsigned v_page_bytes = (unsigned)a.n_v_heads * (unsigned)a.page_size * v_row_bytes;
   const char* const v_head = reinterpret_cast<const char*>(a.v_pages) + ((size_t)(kvh % a.n_v_heads) * a.page_size * a.v_pitch + a.v_offset) * 2;
@@ -488,6 +509,38 @@ __global__ void __launch_bounds__(GROUPS * kWaves * kWave, GROUPS == 1 ? 2 : 1) 
           for (int r = 0; r < 4; ++r) c[i][sub][r] = (c[i][sub][r] - first) + col_slope[i] * (float)(16 * sub + r);
       }
     }
+    if constexpr (TABLE) {
+      // distances of the tile's keys from the block's queries (the same decision for all waves of the block)
+      const int nearest = pos0 + q0 - (base + KT - 1), farthest = pos0 + q_last - base;
+      if (nearest >= a.dist_len - 1) {
+#pragma unroll
+        for (int i = 0; i < NC; ++i)
+#pragma unroll
+          for (int sub = 0; sub < NS; ++sub)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) c[i][sub][r] += col_far[i];
+      } else if (a.dist_pitch > 0 && nearest >= 0 && farthest < a.dist_len) {
+#pragma unroll
+        for (int i = 0; i < NC; ++i) {
+          // (a column that stands for nothing reads the table's start)
+          const float* at = dist_l + (col_ok[i] ? col_row[i] + col_pos[i] - base - 4 * g4 - (KT - 1) : 0);
+#pragma unroll
+          for (int sub = 0; sub < NS; ++sub)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) c[i][sub][r] += at[KT - 1 - 16 * sub - r];
+        }
+      } else {
+#pragma unroll
+        for (int i = 0; i < NC; ++i)
+#pragma unroll
+          for (int sub = 0; sub < NS; ++sub)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const int n = max(min(col_pos[i] - base - 4 * g4 - 16 * sub - r, a.dist_len - 1), 0);
+              c[i][sub][r] += a.dist_pitch > 0 ? dist_l[col_row[i] + n] : a.dist[col_row[i] + n] * a.inv_scale;
+            }
+      }
+    }
     if (kept_of(step) || base + KT - 1 > pos0 + q0 || (WINDOWED && base < window_lo(pos0 + q_last))) mask(base, kept_of(step));
     softmax(pb, alpha, moved);
     output(v_tile(step - 1), pb_prev);
@@ -584,12 +637,18 @@ TL_EXPORT int tl_attn_prefill(const void* q, int q_stride, void* out, int out_st
                               const int32_t* tile_q0, int n_tiles, int n_q_heads, int n_kv_heads, int head_dim,
                               int page_size, int window, float scale, int key_groups, float softcap, int chunk,
                               const float* sinks, int keep_first, int n_v_heads, int v_pitch, int v_offset, int out_pitch,
-                              int out_offset, const float* slopes, hipStream_t stream) {
+                              int out_offset, const float* slopes, const float* dist, int dist_len, int n_k_heads,
+                              hipStream_t stream) {
   if (head_dim != DH) return variant_fail(TL_ERR_ARG, "attn_prefill: built for head_dim %d, called with %d", DH, head_dim);
   if (n_tiles < 0 || n_q_heads <= 0 || n_kv_heads <= 0 || page_size <= 0 || bt_stride <= 0 || window < 0 || chunk < 0 || softcap < 0)
     return variant_fail(TL_ERR_ARG, "attn_prefill: bad sizes");
   if (n_q_heads % n_kv_heads) return variant_fail(TL_ERR_ARG, "attn_prefill: %d query heads are not a multiple of %d kv heads", n_q_heads, n_kv_heads);
   if (n_v_heads <= 0) n_v_heads = n_kv_heads;
+  if (n_k_heads <= 0) n_k_heads = n_kv_heads;
+  if (n_kv_heads % n_k_heads || (dist && dist_len <= 0))
+    return variant_fail(TL_ERR_ARG, "attn_prefill: heads of the key pages, or a table by distance, that do not fit");
+  if (dist && (slopes || softcap > 0 || (keep_first > 0 && (window > 0 || chunk > 0))))
+    return variant_fail(TL_ERR_UNSUPPORTED, "attn_prefill: a table by distance together with slopes, capped scores or kept first keys is not built");
   if (v_pitch <= 0) v_pitch = DH;
   if (out_pitch <= 0) out_pitch = DH;
   if (keep_first < 0 || n_kv_heads % n_v_heads || v_offset < 0 || v_offset + DH > v_pitch || out_offset < 0 || out_offset + DH > out_pitch
@@ -624,22 +683,29 @@ TL_EXPORT int tl_attn_prefill(const void* q, int q_stride, void* out, int out_st
                         page_size, kRowsPerLoad, DH);
   a.scale_log2e = scale * 1.4426950408889634f;
   a.chunk = chunk; a.sinks = sinks; a.slopes = slopes; a.inv_scale = 1.0f / scale;
+  a.dist = dist; a.dist_len = dist_len; a.n_k_heads = n_k_heads;
+  // the heads' rows of the table go to LDS where they leave room for two blocks a CU (16 banks apart)
+  a.dist_pitch = dist ? (dist_len + 47) / 64 * 64 + 16 : 0;
+  if ((size_t)R * a.dist_pitch * sizeof(float) > 16 * 1024) a.dist_pitch = 0;
+  const size_t lds = (size_t)R * a.dist_pitch * sizeof(float);
   a.cap_over_scale = softcap > 0 ? softcap / scale : 0.f;
   a.two_scale_over_cap_log2e = softcap > 0 ? 2.0f * scale / softcap * 1.4426950408889634f : 0.f;
   dim3 grid(n_kv_heads, n_tiles);  // consecutive blocks share a query tile: their loads of q overlap
-  const int mode = slopes ? (softcap > 0 ? 5 : 4) : softcap > 0 ? 2 : a.keep_first > 0 ? 3 : (window > 0 || chunk > 0) ? 1 : 0;
+  const int mode = dist ? 6 : slopes ? (softcap > 0 ? 5 : 4) : softcap > 0 ? 2 : a.keep_first > 0 ? 3 : (window > 0 || chunk > 0) ? 1 : 0;
   const int threads = kWaves * kWave;
 #define TL_PREFILL_LAUNCH(rp)                                                                      \
   do {                                                                                             \
     if (key_groups == 2) {                                                                         \
-      if (mode == 5) attn_prefill_kernel<rp, 5, 2><<<grid, 2 * threads, 0, stream>>>(a);           \
+      if (mode == 6) attn_prefill_kernel<rp, 6, 2><<<grid, 2 * threads, lds, stream>>>(a);         \
+      else if (mode == 5) attn_prefill_kernel<rp, 5, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else if (mode == 4) attn_prefill_kernel<rp, 4, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else if (mode == 2) attn_prefill_kernel<rp, 2, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else if (mode == 3) attn_prefill_kernel<rp, 3, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else if (mode == 1) attn_prefill_kernel<rp, 1, 2><<<grid, 2 * threads, 0, stream>>>(a);      \
       else attn_prefill_kernel<rp, 0, 2><<<grid, 2 * threads, 0, stream>>>(a);                     \
     } else {                                                                                       \
-      if (mode == 5) attn_prefill_kernel<rp, 5, 1><<<grid, threads, 0, stream>>>(a);               \
+      if (mode == 6) attn_prefill_kernel<rp, 6, 1><<<grid, threads, lds, stream>>>(a);             \
+      else if (mode == 5) attn_prefill_kernel<rp, 5, 1><<<grid, threads, 0, stream>>>(a);          \
       else if (mode == 4) attn_prefill_kernel<rp, 4, 1><<<grid, threads, 0, stream>>>(a);          \
       else if (mode == 2) attn_prefill_kernel<rp, 2, 1><<<grid, threads, 0, stream>>>(a);          \
       else if (mode == 3) attn_prefill_kernel<rp, 3, 1><<<grid, threads, 0, stream>>>(a);          \

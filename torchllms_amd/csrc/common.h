@@ -44,6 +44,12 @@ __device__ __forceinline__ T from_f32(float v) {
   return static_cast<T>(v);
 }
 
+// A gate between limits: g sigmoid(slope g) (u + 1) of g = min(gate, limit) and u = up between -limit and limit.
+__device__ __forceinline__ float limited_gate(float gate, float up, float limit, float slope) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.0f + expf(-slope * g)) * (u + 1.0f);
+}
+
 // Sum over the 64 lanes of a wave in a fixed butterfly order; every lane gets the result.
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll

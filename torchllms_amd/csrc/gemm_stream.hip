@@ -62,7 +62,8 @@ __device__ __forceinline__ float gate_activation(float g, int act) {
 }
 
 struct NormArgs {
-  int act;  // kGated, kGatedHalf: the gate's activation (see gate_activation)
+  int act;  // kGated, kGatedHalf: the gate's activation (see gate_activation); 2: a gate between limits (limited_gate)
+  float limit, slope;  // act 2
   // kGated, kGatedHalf, kQkv: the rows of A are to be read as A[m] / sqrt(sum[m] / width + eps);
   // row_sums [n_row_sums][16] are pieces of sum[m] (piece by piece, the 16 rows side by side).  Null: A as it is.
   const float* row_sums;
@@ -345,6 +346,10 @@ gemm_stream_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __restri
         if (n >= N) continue;
         const float g = to_f32(from_f32<OutT>(acc[0][i]));
         const float u = to_f32(from_f32<OutT>(up[i]));
+        if (na.act == 2) {  // (uniform)
+          C[(size_t)n16 * ldc + n] = from_f32<OutT>(limited_gate(g, u, na.limit, na.slope));
+          continue;
+        }
         const float act = to_f32(from_f32<OutT>(gate_activation(g, na.act)));
         C[(size_t)n16 * ldc + n] = from_f32<OutT>(act * u);
       }
@@ -382,6 +387,10 @@ gemm_stream_kernel(const bf16_t* __restrict__ A, int lda, const bf16_t* __restri
       if constexpr (GLU) {
         const float g = to_f32(from_f32<OutT>(acc[0][i]));
         const float u = to_f32(from_f32<OutT>(acc[1][i]));
+        if (na.act == 2) {  // (uniform)
+          C[(size_t)n16 * ldc + n] = from_f32<OutT>(limited_gate(g, u, na.limit, na.slope));
+          continue;
+        }
         const float act = to_f32(from_f32<OutT>(gate_activation(g, na.act)));
         C[(size_t)n16 * ldc + n] = from_f32<OutT>(act * u);
       } else {
@@ -487,16 +496,18 @@ TL_EXPORT int tl_gemm_stream(const void* A, int lda, const void* W, int ldw, voi
 
 // The gated pair of products: W [2 N, K] = gate rows | up rows; C [M, N] bfloat16 =
 // act(A gate^T) * (A up^T), act = silu (0) or the tanh form of gelu (1), rounded as the two products, the
-// activation and the final product would be if each were stored in bfloat16.  cols: 16 or 8 columns of C per block.
+// activation and the final product would be if each were stored in bfloat16; act 2: the gate between limits
+// (limit, slope; see limited_gate) of the two products rounded to bfloat16.  cols: 16 or 8 columns of C per block.
 // row_sums [n_row_sums][16] 32-bit or null: pieces of a sum of squares per row, as tl_gemm_stream_residual
 // leaves them; then row m of both products is scaled by 1 / sqrt(sum / K + eps) before the roundings.
 TL_EXPORT int tl_gemm_stream_glu(const void* A, int lda, const void* W, int ldw, void* C, int ldc, int M, int N,
                                  int K, int waves, int cols, const float* row_sums, int n_row_sums, float eps,
-                                 int act, hipStream_t stream) {
+                                 int act, float limit, float slope, hipStream_t stream) {
   TL_REQUIRE(cols == 8 || cols == 16, "gemm_stream_glu: cols must be 8 or 16");
-  TL_REQUIRE(act == 0 || act == 1, "gemm_stream_glu: activation %d (0: silu, 1: gelu_tanh)", act);
+  TL_REQUIRE(act >= 0 && act <= 2, "gemm_stream_glu: activation %d (0: silu, 1: gelu_tanh, 2: between limits)", act);
+  TL_REQUIRE(act != 2 || limit > 0.f, "gemm_stream_glu: a limit that is not positive");
   NormArgs na = {};
-  na.act = act;
+  na.act = act; na.limit = limit; na.slope = slope;
   na.row_sums = row_sums; na.n_row_sums = n_row_sums; na.width = (float)K; na.eps = eps;
   return run(A, lda, W, ldw, C, ldc, M, N, K, TL_BF16, waves, cols == 8 ? kGatedHalf : kGated, QkvArgs{}, na, stream);
 }

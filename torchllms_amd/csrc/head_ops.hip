@@ -311,6 +311,137 @@ rmsnorm_columns_kernel(const XT* __restrict__ x, int x_stride, const int32_t* __
   }
 }
 
+// ----------------------------------------------------------------------------- a branch into the stream, and a norm
+// For output row r (row s = rows ? rows[r] : r of stream and branch):  h = stream[s] + branch[s], in 32-bit;
+// y[r] = T(h / sqrt(mean(h^2) + eps) * w).  Without a row gather the stream becomes h.  The branch is a tensor of DT, or
+// (partial given) the 32-bit slices of a product split along K, added in their order.
+template <typename DT>
+struct AddNormArgs {
+  float* stream;
+  const DT* branch;
+  const float* partial;
+  int splits;
+  size_t split_stride;
+  const int32_t* rows;
+  const float* w;
+  float eps;
+  int hidden;
+};
+
+template <typename T> struct alignas(4 * sizeof(T)) FourOf { T e[4]; };
+
+// Rows of a multiple of four elements (up to 4 * CH of them a thread), held in registers: everything a thread needs is
+// asked for at once.  A row's sum has an order that its width alone decides.
+template <typename DT, typename T, int CH, int THREADS>
+__global__ void __launch_bounds__(THREADS) add_norm_held_kernel(const AddNormArgs<DT> a, T* __restrict__ y) {
+#pragma clang fp contract(off)
+  __shared__ float scratch[THREADS / kWave];
+  const size_t r = blockIdx.x;
+  const size_t s = a.rows ? (size_t)a.rows[r] : r;
+  const int n_waves = blockDim.x / kWave;
+  float* sr = a.stream + s * a.hidden;
+  FourOf<float> h[CH], w[CH], part[CH];
+  FourOf<DT> b[CH];
+  int at[CH];
+  bool in[CH];
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    const int i = 4 * ((int)threadIdx.x + c * (int)blockDim.x);
+    in[c] = i < a.hidden;
+    at[c] = in[c] ? i : 0;  // (elements past the end are the row's first once more, and not used)
+    h[c] = *reinterpret_cast<const FourOf<float>*>(sr + at[c]);
+    w[c] = *reinterpret_cast<const FourOf<float>*>(a.w + at[c]);
+    if (a.partial) part[c] = *reinterpret_cast<const FourOf<float>*>(a.partial + s * a.hidden + at[c]);  // (uniform)
+    else b[c] = *reinterpret_cast<const FourOf<DT>*>(a.branch + s * a.hidden + at[c]);
+  }
+  if (a.partial) {
+    for (int k = 1; k < a.splits; ++k) {
+      FourOf<float> next[CH];
+#pragma unroll
+      for (int c = 0; c < CH; ++c) next[c] = *reinterpret_cast<const FourOf<float>*>(a.partial + k * a.split_stride + s * a.hidden + at[c]);
+#pragma unroll
+      for (int c = 0; c < CH; ++c)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) part[c].e[e] += next[c].e[e];
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < CH; ++c)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      h[c].e[e] += a.partial ? part[c].e[e] : to_f32(b[c].e[e]);
+      if (in[c]) ss += h[c].e[e] * h[c].e[e];
+    }
+  ss = wave_sum(ss);
+  if (threadIdx.x % kWave == 0) scratch[threadIdx.x / kWave] = ss;
+  __syncthreads();
+  ss = 0.f;
+  for (int i = 0; i < n_waves; ++i) ss += scratch[i];
+  const float inv = 1.0f / sqrtf(ss / (float)a.hidden + a.eps);
+#pragma unroll
+  for (int c = 0; c < CH; ++c) {
+    if (!in[c]) continue;
+    FourOf<T> o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o.e[e] = from_f32<T>(h[c].e[e] * inv * w[c].e[e]);
+    *reinterpret_cast<FourOf<T>*>(y + r * a.hidden + at[c]) = o;
+    if (!a.rows) *reinterpret_cast<FourOf<float>*>(sr + at[c]) = h[c];
+  }
+}
+
+// Rows of any width that fit the LDS.
+template <typename DT, typename T>
+__global__ void __launch_bounds__(kRowThreads) add_norm_kernel(const AddNormArgs<DT> a, T* __restrict__ y) {
+#pragma clang fp contract(off)
+  __shared__ float scratch[kRowThreads / kWave];
+  extern __shared__ __attribute__((aligned(16))) float row_l[];
+  const size_t r = blockIdx.x;
+  const size_t s = a.rows ? (size_t)a.rows[r] : r;
+  float* sr = a.stream + s * a.hidden;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < a.hidden; i += kRowThreads) {
+    float d = 0.f;
+    if (a.partial) {
+      d = a.partial[s * a.hidden + i];
+      for (int k = 1; k < a.splits; ++k) d += a.partial[k * a.split_stride + s * a.hidden + i];
+    } else {
+      d = to_f32(a.branch[s * a.hidden + i]);
+    }
+    const float h = sr[i] + d;
+    row_l[i] = h;
+    ss += h * h;
+  }
+  ss = block_sum<kRowThreads / kWave>(ss, scratch);
+  const float inv = 1.0f / sqrtf(ss / (float)a.hidden + a.eps);
+  for (int i = threadIdx.x; i < a.hidden; i += kRowThreads) {
+    y[r * a.hidden + i] = from_f32<T>(row_l[i] * inv * a.w[i]);
+    if (!a.rows) sr[i] = row_l[i];
+  }
+}
+
+template <typename DT, typename T>
+int launch_add_norm(const AddNormArgs<DT>& a, T* y, int n, hipStream_t stream) {
+  const int fours = a.hidden / 4;
+  const uintptr_t places = (uintptr_t)a.stream | (uintptr_t)a.w | (uintptr_t)a.partial;
+  if (a.hidden % 4 == 0 && fours <= 4096 && places % 16 == 0 && a.split_stride % 4 == 0 && (uintptr_t)a.branch % (4 * sizeof(DT)) == 0 &&
+      (uintptr_t)y % (4 * sizeof(T)) == 0) {
+    if (fours <= 256) add_norm_held_kernel<DT, T, 1, 256><<<n, (fours + kWave - 1) / kWave * kWave, 0, stream>>>(a, y);
+    else if (fours <= 512) add_norm_held_kernel<DT, T, 2, 256><<<n, 256, 0, stream>>>(a, y);
+    else if (fours <= 1024) add_norm_held_kernel<DT, T, 4, 256><<<n, 256, 0, stream>>>(a, y);
+    else add_norm_held_kernel<DT, T, 4, 1024><<<n, (fours + 4 * kWave - 1) / (4 * kWave) * kWave, 0, stream>>>(a, y);
+    return tl_check_launch("add_norm");
+  }
+  const size_t lds = (size_t)a.hidden * sizeof(float);
+  if (lds + 64 > (size_t)tl_device_facts().lds_bytes) return tl_fail(TL_ERR_UNSUPPORTED, "add_norm: rows of %d elements do not fit the LDS", a.hidden);
+  if (lds > 48 * 1024) {
+    hipError_t e = hipFuncSetAttribute((const void*)add_norm_kernel<DT, T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return tl_fail(TL_ERR_HIP, "add_norm: %s", hipGetErrorString(e));
+  }
+  add_norm_kernel<DT, T><<<n, kRowThreads, lds, stream>>>(a, y);
+  return tl_check_launch("add_norm");
+}
+
 // ----------------------------------------------------------------------------- gates, packing, cap
 // x[t, c] *= sigmoid(g[t, c / per]) for c < width: per = 1 gates channel by channel, per = the head size gates
 // head by head.
@@ -475,6 +606,23 @@ TL_EXPORT int tl_rmsnorm_columns(const void* x, int x_stride, int x_dtype, const
   else return tl_fail(TL_ERR_ARG, "rmsnorm_columns: input dtype %d with output dtype %d", x_dtype, y_dtype);
 #undef TL_NORM
   return tl_check_launch("rmsnorm_columns");
+}
+
+// branch [.., hidden] of branch_dtype, or partial: slice k of row s at partial + k * split_stride + s * hidden.
+TL_EXPORT int tl_add_norm(float* stream_rows, const void* branch, int branch_dtype, const float* partial, int splits, long long split_stride,
+                          const int32_t* rows, const float* w, float eps, void* y, int n, int hidden, int y_dtype, hipStream_t stream) {
+  TL_REQUIRE(n >= 0 && hidden > 0, "add_norm: bad sizes");
+  TL_REQUIRE((branch == nullptr) != (partial == nullptr), "add_norm: a branch, or the slices of one");
+  TL_REQUIRE(partial == nullptr || (splits >= 1 && split_stride >= 0), "add_norm: bad slices");
+  if (n == 0) return TL_OK;
+#define TL_ADD(DT, T)                                                                                                                   \
+  return launch_add_norm<DT, T>({stream_rows, (const DT*)branch, partial, splits, (size_t)split_stride, rows, w, eps, hidden}, (T*)y, n, stream)
+  const bool wide = partial != nullptr || branch_dtype == TL_F32;  // (slices: the branch's type does not matter)
+  if (y_dtype == TL_F32 && wide) TL_ADD(float, float);
+  if (y_dtype == TL_BF16 && wide) TL_ADD(float, bf16_t);
+  if (y_dtype == TL_BF16 && branch_dtype == TL_BF16) TL_ADD(bf16_t, bf16_t);
+#undef TL_ADD
+  return tl_fail(TL_ERR_ARG, "add_norm: a branch of dtype %d with results of dtype %d", branch_dtype, y_dtype);
 }
 
 TL_EXPORT int tl_sigmoid_gate(void* x, int x_stride, const void* g, int g_stride, int n, int width, int per, int dtype,

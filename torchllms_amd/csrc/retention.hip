@@ -6,7 +6,7 @@
 // (H * dv each) are read from their offsets.  cos_sin: the step's table [n_tokens][rot / 2][2] (channel i of a head is
 // paired with channel i + rot / 2; channels from rot on pass).  Rotated keys and queries, decays, sums, state and norm
 // are 32-bit.
-#include "common.h"
+#include "recurrence.h"
 
 namespace {
 
@@ -27,23 +27,6 @@ struct RetentionArgs {
   float eps, k_scale;
 };
 
-__device__ __forceinline__ float lane_xor1(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xf, 0xf, false));
-}
-__device__ __forceinline__ float lane_xor2(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x4E, 0xf, 0xf, false));
-}
-__device__ __forceinline__ float lane_half_mirror(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0x141, 0xf, 0xf, false));
-}
-// The sum over eight neighbouring lanes; each of them gets the same bits.
-__device__ __forceinline__ float sum_of_eight_lanes(float v) {
-  v += lane_xor1(v);
-  v += lane_xor2(v);
-  v += lane_half_mirror(v);
-  return v;
-}
-
 // Element i of a head after the rotation, from the head's row in the projection (x) and the token's table (cs).
 template <typename T>
 __device__ __forceinline__ float rotated(const T* x, const float* cs, int rot, int i) {
@@ -59,7 +42,6 @@ __device__ __forceinline__ float rotated(const T* x, const float* cs, int rot, i
 
 // Four consecutive elements i .. i + 3 of a head after the rotation (rot a multiple of 8, rows aligned to four
 // elements: the four lie in one half, and so do their partners), the same bits as `rotated`.
-template <typename T> struct alignas(4 * sizeof(T)) Four { T e[4]; };
 template <typename T>
 __device__ __forceinline__ void rotated_four(const T* x, const float* cs, int rot, int i, float (&out)[4]) {
 #pragma clang fp contract(off)
@@ -310,10 +292,6 @@ int launch_walk(const RetentionArgs<T>& a, int n_seqs, int n_tokens, hipStream_t
 // other operand of (P V)[t][j], so they stay in their registers.
 constexpr int kSeg = 64;
 constexpr int kChunkThreads = 256;
-typedef float f32x4_t __attribute__((ext_vector_type(4)));
-
-__device__ __forceinline__ f32x4_t mfma_f32(float a, float b, f32x4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-
 // decay^n for n = 0 .. kSeg into LDS, by the first threads of the block.
 __device__ __forceinline__ void fill_powers(float* pw, float decay) {
   if (threadIdx.x <= kSeg) pw[threadIdx.x] = powf(decay, (float)threadIdx.x);

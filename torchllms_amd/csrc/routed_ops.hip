@@ -13,12 +13,13 @@ __device__ __forceinline__ float sigmoid_r(float z) { return 1.0f / (1.0f + expf
 // largest of s + correction are chosen (of equal ones the lower index), and the weights are their s.
 // correction may be null, and so may bias, which is added to z first (32-bit).  n_groups > 0: the outputs form that many equal groups of neighbours, a group's score is
 // the largest s in it, and only outputs of the keep_groups best groups (of equal ones the lower) can be chosen.
-// normalize: the weights are divided by their sum (+ 1e-20); then they are multiplied by route_scale.
+// normalize: the weights are divided by their sum (+ 1e-20); then they are multiplied by route_scale.  sigmoid: s is the
+// logistic function of every z by itself instead of the softmax over all.
 constexpr int kRouterPerLane = 8;  // outputs a lane holds: up to 512 experts
 __global__ void __launch_bounds__(256)
 router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __restrict__ correction, int n, int n_out, int top,
                    int32_t* __restrict__ ids, float* __restrict__ weights, int n_groups, int keep_groups, int normalize,
-                   float route_scale, const float* __restrict__ bias) {
+                   float route_scale, const float* __restrict__ bias, int sigmoid) {
   const int t = blockIdx.x * (blockDim.x / kWave) + threadIdx.x / kWave;
   const int lane = threadIdx.x % kWave;
   if (t >= n) return;
@@ -36,14 +37,14 @@ router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __res
 #pragma unroll
   for (int u = 0; u < kRouterPerLane; ++u) {
     const int e = lane + u * kWave;
-    s[u] = e < n_out ? expf(s[u] - mx) : 0.f;
+    s[u] = e < n_out ? (sigmoid ? sigmoid_r(s[u]) : expf(s[u] - mx)) : 0.f;
     sum += s[u];
   }
   sum = wave_sum(sum);
 #pragma unroll
   for (int u = 0; u < kRouterPerLane; ++u) {
     const int e = lane + u * kWave;
-    s[u] = s[u] / sum;
+    s[u] = sigmoid ? s[u] : s[u] / sum;
     c[u] = e < n_out ? (correction ? s[u] + correction[e] : s[u]) : -INFINITY;
   }
   if (n_groups > 0) {
@@ -399,10 +400,10 @@ __global__ void expert_offsets_kernel(const int32_t* __restrict__ counts, int n_
 
 // A block a pair: the pair takes the next free row of its expert's range (which of an expert's pairs gets which row
 // depends on timing; a row's result does not depend on where it lies), remembers it in pos[p], and its token's row of
-// x is copied there.
+// x is copied there (times weights[p] where they are given: routers that weigh an expert's input).
 template <typename T>
 __global__ void __launch_bounds__(256)
-expert_gather_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, const int32_t* __restrict__ offsets,
+expert_gather_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, const float* __restrict__ weights, const int32_t* __restrict__ offsets,
                      int32_t* __restrict__ cursor, int top, int32_t* __restrict__ pos, T* __restrict__ rows, int D) {
   __shared__ int at_l;
   const int p = blockIdx.x;
@@ -414,11 +415,26 @@ expert_gather_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, c
   __syncthreads();
   const T* src = x + (size_t)(p / top) * D;
   T* dst = rows + (size_t)at_l * D;
-  for (int d = threadIdx.x; d < D; d += blockDim.x) dst[d] = src[d];
+  if (weights) {
+    const float w = weights[p];
+    for (int d = threadIdx.x; d < D; d += blockDim.x) dst[d] = from_f32<T>(w * to_f32(src[d]));
+  } else {
+    for (int d = threadIdx.x; d < D; d += blockDim.x) dst[d] = src[d];
+  }
+}
+
+// out[p, d] = T(weights[p] * x[p / top, d]): the pairs' inputs in their own order.
+template <typename T>
+__global__ void __launch_bounds__(256)
+pair_rows_kernel(const T* __restrict__ x, const float* __restrict__ weights, T* __restrict__ out, int top, int D) {
+  const int p = blockIdx.x;
+  const int d = blockIdx.y * blockDim.x + threadIdx.x;
+  if (d < D) out[(size_t)p * D + d] = from_f32<T>(weights[p] * to_f32(x[(size_t)(p / top) * D + d]));
 }
 
 // out[t, d] = T(sum_j w[t, j] * (e_j < n_experts ? y[pos[t, j], d] : x[t, d]) + sigmoid(sg[t]) * shared[t, d]): the
-// experts' results (32-bit, or of the tensors' dtype) back in the order of the tokens, weighted and added in the order of a token's choices.
+// experts' results (32-bit, or of the tensors' dtype) back in the order of the tokens, weighted (weights null: as they are) and added
+// in the order of a token's choices.
 template <typename T, typename YT>
 __global__ void __launch_bounds__(256)
 expert_combine_kernel(const YT* __restrict__ y, const int32_t* __restrict__ pos, const int32_t* __restrict__ ids,
@@ -433,7 +449,7 @@ expert_combine_kernel(const YT* __restrict__ y, const int32_t* __restrict__ pos,
   float total = 0.f;
   for (int j = 0; j < top; ++j) {
     const int e = ids[(size_t)t * top + j];
-    const float wj = weights[(size_t)t * top + j];
+    const float wj = weights ? weights[(size_t)t * top + j] : 1.f;
     total += wj * (e < n_experts ? to_f32(y[(size_t)pos[(size_t)t * top + j] * D + d]) : to_f32(x[(size_t)t * D + d]));
   }
   if (shared) total += share * to_f32(shared[(size_t)t * D + d]);
@@ -683,7 +699,7 @@ __global__ void __launch_bounds__(256) relu_square_kernel(T* __restrict__ x, siz
 // ============================================================================= C interface
 TL_EXPORT int tl_router_topk(const float* z, int z_stride, const float* correction, int n, int n_out, int top, int32_t* ids,
                              float* weights, int n_groups, int keep_groups, int normalize, float route_scale, const float* bias,
-                             hipStream_t stream) {
+                             int sigmoid, hipStream_t stream) {
   TL_REQUIRE(n >= 0 && n_out > 0 && top > 0 && top <= n_out && z_stride >= n_out, "router_topk: bad sizes");
   TL_REQUIRE(n_groups >= 0 && (n_groups == 0 || (n_groups <= kWave && n_out % n_groups == 0 && keep_groups > 0 && keep_groups <= n_groups
                                                  && (long long)keep_groups * (n_out / n_groups) >= top)),
@@ -693,7 +709,7 @@ TL_EXPORT int tl_router_topk(const float* z, int z_stride, const float* correcti
   if (n == 0) return TL_OK;
   const int per_block = 256 / kWave;
   router_topk_kernel<<<(n + per_block - 1) / per_block, 256, 0, stream>>>(z, z_stride, correction, n, n_out, top, ids, weights, n_groups,
-                                                                         keep_groups, normalize, route_scale, bias);
+                                                                         keep_groups, normalize, route_scale, bias, sigmoid);
   return tl_check_launch("router_topk");
 }
 
@@ -771,7 +787,8 @@ TL_EXPORT int tl_expert_down_rows(const void* mid, const void* w_d, const int32_
 }
 
 // counts, cursor: n_out int32 each (counts zeroed by the caller); offsets: n_out + 1; pos: n * top; rows [n * top, D].
-TL_EXPORT int tl_expert_gather(const void* x, const int32_t* ids, int n, int top, int n_out, int32_t* counts, int32_t* offsets,
+// weights [n * top] or null: a pair's row is its token's times its weight.
+TL_EXPORT int tl_expert_gather(const void* x, const int32_t* ids, const float* weights, int n, int top, int n_out, int32_t* counts, int32_t* offsets,
                                int32_t* cursor, int32_t* pos, void* rows, int D, int dtype, hipStream_t stream) {
   TL_REQUIRE(n >= 0 && top > 0 && n_out > 0 && D > 0, "expert_gather: bad sizes");
   TL_REQUIRE((long long)n * top <= 0x7fffffff, "expert_gather: too many pairs a step");
@@ -780,9 +797,20 @@ TL_EXPORT int tl_expert_gather(const void* x, const int32_t* ids, int n, int top
   const int pairs = n * top;
   expert_count_kernel<<<(pairs + 255) / 256 < 1024 ? (pairs + 255) / 256 : 1024, 256, 0, stream>>>(ids, pairs, counts);
   expert_offsets_kernel<<<1, 64, 0, stream>>>(counts, n_out, offsets, cursor);
-  if (dtype == TL_F32) expert_gather_kernel<float><<<pairs, 256, 0, stream>>>((const float*)x, ids, offsets, cursor, top, pos, (float*)rows, D);
-  else expert_gather_kernel<bf16_t><<<pairs, 256, 0, stream>>>((const bf16_t*)x, ids, offsets, cursor, top, pos, (bf16_t*)rows, D);
+  if (dtype == TL_F32) expert_gather_kernel<float><<<pairs, 256, 0, stream>>>((const float*)x, ids, weights, offsets, cursor, top, pos, (float*)rows, D);
+  else expert_gather_kernel<bf16_t><<<pairs, 256, 0, stream>>>((const bf16_t*)x, ids, weights, offsets, cursor, top, pos, (bf16_t*)rows, D);
   return tl_check_launch("expert_gather");
+}
+
+// out [n * top, D]: the pairs in their own order, each its token's row of x times its weight.
+TL_EXPORT int tl_pair_rows(const void* x, const float* weights, void* out, int n, int top, int D, int dtype, hipStream_t stream) {
+  TL_REQUIRE(n >= 0 && top > 0 && D > 0 && (long long)n * top <= 0x7fffffff && (D + 255) / 256 <= 65535, "pair_rows: bad sizes");
+  if (n == 0) return TL_OK;
+  const dim3 grid(n * top, (D + 255) / 256);
+  if (dtype == TL_F32) pair_rows_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, weights, (float*)out, top, D);
+  else if (dtype == TL_BF16) pair_rows_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, weights, (bf16_t*)out, top, D);
+  else return tl_fail(TL_ERR_ARG, "pair_rows: unknown dtype %d", dtype);
+  return tl_check_launch("pair_rows");
 }
 
 // y: the experts' results in the order of the gathered rows, 32-bit (y_f32) or of the tensors' dtype.

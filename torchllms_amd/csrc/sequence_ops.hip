@@ -26,14 +26,39 @@ __device__ __forceinline__ float group_sum(float v, int width) {
 }
 
 // ----------------------------------------------------------------------------- scaled embedding
-// out[t, :] = float(table[tokens[t], :]) * scale, 32-bit.
-template <typename T>
+// out[t, :] = float(table[tokens[t], :]) * scale, 32-bit, plus float(pos_table[positions[t], :]) where a table of
+// position vectors is given.  V elements a load.
+template <typename T, int V>
 __global__ void embed_scaled_kernel(const int32_t* __restrict__ tokens, const T* __restrict__ table,
-                                    float* __restrict__ out, int hidden, float scale) {
+                                    float* __restrict__ out, int hidden, float scale, const int32_t* __restrict__ positions,
+                                    const T* __restrict__ pos_table) {
+#pragma clang fp contract(off)
+  struct alignas(sizeof(T) * V) Vec { T e[V]; };
+  struct alignas(sizeof(float) * V) OutVec { float e[V]; };
   const int t = blockIdx.x;
   const T* src = table + (size_t)tokens[t] * hidden;
+  const T* pos = pos_table ? pos_table + (size_t)positions[t] * hidden : nullptr;
   float* dst = out + (size_t)t * hidden;
-  for (int i = threadIdx.x; i < hidden; i += blockDim.x) dst[i] = to_f32(src[i]) * scale;
+  for (int i = threadIdx.x * V; i < hidden; i += blockDim.x * V) {
+    const Vec a = *reinterpret_cast<const Vec*>(src + i);
+    const Vec b = *reinterpret_cast<const Vec*>((pos ? pos : src) + i);
+    OutVec o;
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      o.e[e] = to_f32(a.e[e]) * scale;
+      if (pos) o.e[e] += to_f32(b.e[e]);
+    }
+    *reinterpret_cast<OutVec*>(dst + i) = o;
+  }
+}
+
+template <typename T>
+int embed_scaled_launch(const int32_t* tokens, const T* table, float* out, int n, int hidden, float scale, const int32_t* positions,
+                        const T* pos_table, hipStream_t stream) {
+  const bool fours = hidden % 4 == 0 && (uintptr_t)table % (4 * sizeof(T)) == 0 && (uintptr_t)pos_table % (4 * sizeof(T)) == 0 && (uintptr_t)out % 16 == 0;
+  if (fours) embed_scaled_kernel<T, 4><<<n, 256, 0, stream>>>(tokens, table, out, hidden, scale, positions, pos_table);
+  else embed_scaled_kernel<T, 1><<<n, 256, 0, stream>>>(tokens, table, out, hidden, scale, positions, pos_table);
+  return tl_check_launch("embed_scaled");
 }
 
 // ----------------------------------------------------------------------------- layer norm
@@ -96,10 +121,11 @@ int layernorm_launch(const void* x, const void* d0, const void* d1, float mult, 
 }
 
 // ----------------------------------------------------------------------------- gated activation
-// gate_up: [n, 2F] = gate | up.  out[n, F] = T(act(float(gate)) * float(up)); act 1: gelu in its tanh form.
+// gate_up: [n, 2F] = gate | up.  ACT 1: out[n, F] = T(gelu(gate) * up), gelu in its tanh form; ACT 2, a gate between
+// limits: g = min(gate, limit), u = up between -limit and limit, out[n, F] = T(g / (1 + exp(-slope g)) * (u + 1)).
 // A thread takes V consecutive columns of one row (V elements = 16 bytes when the row allows it).
-template <typename T, int V>
-__global__ void gelu_mul_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int n, int inter) {
+template <typename T, int V, int ACT>
+__global__ void gate_mul_kernel(const T* __restrict__ gate_up, T* __restrict__ out, int n, int inter, float limit, float slope) {
   const int c0 = (blockIdx.x * blockDim.x + threadIdx.x) * V;
   if (c0 >= inter) return;
   struct alignas(sizeof(T) * V) Vec { T e[V]; };
@@ -109,20 +135,23 @@ __global__ void gelu_mul_kernel(const T* __restrict__ gate_up, T* __restrict__ o
     const Vec u = *reinterpret_cast<const Vec*>(gp + inter);
     Vec o;
 #pragma unroll
-    for (int i = 0; i < V; ++i) o.e[i] = from_f32<T>(gelu_tanh_f(to_f32(g.e[i])) * to_f32(u.e[i]));
+    for (int i = 0; i < V; ++i) {
+      if constexpr (ACT == 1) o.e[i] = from_f32<T>(gelu_tanh_f(to_f32(g.e[i])) * to_f32(u.e[i]));
+      else o.e[i] = from_f32<T>(limited_gate(to_f32(g.e[i]), to_f32(u.e[i]), limit, slope));
+    }
     *reinterpret_cast<Vec*>(out + (size_t)r * inter + c0) = o;
   }
 }
 
-template <typename T>
-int gelu_mul_launch(const T* gate_up, T* out, int n, int inter, hipStream_t stream) {
+template <typename T, int ACT>
+int gate_mul_launch(const T* gate_up, T* out, int n, int inter, float limit, float slope, hipStream_t stream) {
   constexpr int kVec = 16 / sizeof(T);
   const bool wide = inter % kVec == 0 && ((uintptr_t)gate_up % 16) == 0 && ((uintptr_t)out % 16) == 0;
   const int per_block = 256 * (wide ? kVec : 1);
   const dim3 grid((inter + per_block - 1) / per_block, n < 65535 ? n : 65535);
-  if (wide) gelu_mul_kernel<T, kVec><<<grid, 256, 0, stream>>>(gate_up, out, n, inter);
-  else gelu_mul_kernel<T, 1><<<grid, 256, 0, stream>>>(gate_up, out, n, inter);
-  return tl_check_launch("gelu_mul");
+  if (wide) gate_mul_kernel<T, kVec, ACT><<<grid, 256, 0, stream>>>(gate_up, out, n, inter, limit, slope);
+  else gate_mul_kernel<T, 1, ACT><<<grid, 256, 0, stream>>>(gate_up, out, n, inter, limit, slope);
+  return tl_check_launch("gate_mul");
 }
 
 // ----------------------------------------------------------------------------- rotation, unit norm, cache write
@@ -911,16 +940,15 @@ int launch_head_output(const float* o_raw, const T* gate, int gate_stride, int g
 
 // ============================================================================= C interface
 TL_EXPORT int tl_embed_scaled(const int32_t* tokens, const void* table, float* out, int n_tokens, int hidden, float scale,
-                              int dtype, hipStream_t stream) {
+                              int dtype, const int32_t* positions, const void* pos_table, hipStream_t stream) {
   TL_REQUIRE(n_tokens >= 0 && hidden > 0, "embed_scaled: bad sizes n_tokens=%d hidden=%d", n_tokens, hidden);
+  TL_REQUIRE(pos_table == nullptr || positions != nullptr, "embed_scaled: position vectors without positions");
   if (n_tokens == 0) return TL_OK;
   if (dtype == TL_F32)
-    embed_scaled_kernel<float><<<n_tokens, 256, 0, stream>>>(tokens, (const float*)table, out, hidden, scale);
-  else if (dtype == TL_BF16)
-    embed_scaled_kernel<bf16_t><<<n_tokens, 256, 0, stream>>>(tokens, (const bf16_t*)table, out, hidden, scale);
-  else
-    return tl_fail(TL_ERR_ARG, "embed_scaled: unknown dtype %d", dtype);
-  return tl_check_launch("embed_scaled");
+    return embed_scaled_launch(tokens, (const float*)table, out, n_tokens, hidden, scale, positions, (const float*)pos_table, stream);
+  if (dtype == TL_BF16)
+    return embed_scaled_launch(tokens, (const bf16_t*)table, out, n_tokens, hidden, scale, positions, (const bf16_t*)pos_table, stream);
+  return tl_fail(TL_ERR_ARG, "embed_scaled: unknown dtype %d", dtype);
 }
 
 // x, h_out: [.., hidden] of stream_dtype; d0, d1, y of dtype; w, b 32-bit.  n output rows.
@@ -944,9 +972,17 @@ TL_EXPORT int tl_layernorm(const void* x, const void* d0, const void* d1, float 
 TL_EXPORT int tl_gelu_mul(const void* gate_up, void* out, int n, int inter, int dtype, hipStream_t stream) {
   TL_REQUIRE(n >= 0 && inter > 0, "gelu_mul: bad sizes n=%d inter=%d", n, inter);
   if (n == 0) return TL_OK;
-  if (dtype == TL_F32) return gelu_mul_launch((const float*)gate_up, (float*)out, n, inter, stream);
-  if (dtype == TL_BF16) return gelu_mul_launch((const bf16_t*)gate_up, (bf16_t*)out, n, inter, stream);
+  if (dtype == TL_F32) return gate_mul_launch<float, 1>((const float*)gate_up, (float*)out, n, inter, 0.f, 0.f, stream);
+  if (dtype == TL_BF16) return gate_mul_launch<bf16_t, 1>((const bf16_t*)gate_up, (bf16_t*)out, n, inter, 0.f, 0.f, stream);
   return tl_fail(TL_ERR_ARG, "gelu_mul: unknown dtype %d", dtype);
+}
+
+TL_EXPORT int tl_limited_gate_mul(const void* gate_up, void* out, int n, int inter, float limit, float slope, int dtype, hipStream_t stream) {
+  TL_REQUIRE(n >= 0 && inter > 0 && limit > 0.f, "limited_gate_mul: bad sizes n=%d inter=%d, or a limit that is not positive", n, inter);
+  if (n == 0) return TL_OK;
+  if (dtype == TL_F32) return gate_mul_launch<float, 2>((const float*)gate_up, (float*)out, n, inter, limit, slope, stream);
+  if (dtype == TL_BF16) return gate_mul_launch<bf16_t, 2>((const bf16_t*)gate_up, (bf16_t*)out, n, inter, limit, slope, stream);
+  return tl_fail(TL_ERR_ARG, "limited_gate_mul: unknown dtype %d", dtype);
 }
 
 TL_EXPORT int tl_rope_norm_kv_write(void* qkv, int n_tokens, int n_q, int n_kv, int dk, int dv, const float* cos_sin, int rot,

@@ -35,6 +35,9 @@ def paged_attention(
     keep_first: int = 0,
     value_heads=None,
     slopes=None,
+    distances=None,
+    key_heads=None,
+    out=None,
 ) -> torch.Tensor:
     """Attention of this step's queries (first Hq * dh columns of ``qkv``) over their requests'
     cached keys and values; returns [n_tokens, Hq * dv].  Capped scores (``softcap``), chunks
@@ -42,8 +45,10 @@ def paged_attention(
     channels of the key rows (``values_in_keys``, from ``value_offset`` on), are the plain kernel's alone.  First keys
     that stay visible behind a window (``keep_first``), values with fewer heads than the keys (``value_heads``) and
     values whose head size is a whole multiple of the keys' are every kernel's: the MFMA kernels then take the value
-    channels in calls of one key head size each.  A bias by distance (``slopes``) is every kernel's, together with kept
-    first keys only the plain kernel's and the decode kernel's."""
+    channels in calls of one key head size each.  A bias by distance (``slopes`` or, by table, ``distances``) is every
+    kernel's, together with kept first keys only the plain kernel's and the decode kernel's.  ``key_heads`` (key pages of
+    fewer heads, with ``value_heads``): the MFMA kernels'.  ``out``: row-major [n_tokens, Hq * dv] (some columns of a wider
+    matrix will do) that receives the result."""
     n = qkv.shape[0]
     n_dec = ctx.host.n_decode
     v_dim = head_dim if v_head_dim is None else int(v_head_dim)
@@ -51,15 +56,21 @@ def paged_attention(
     fewer_values = value_heads is not None and value_heads != n_kv_heads
     # (the MFMA kernels take a cap, chunks, sinks, kept first keys and fewer value heads, and values of the keys' head size a call)
     plain_only = values_in_keys or v_dim % head_dim != 0
-    extended = softcap > 0 or chunk > 0 or sinks is not None or plain_only or kept > 0 or fewer_values or v_dim != head_dim or slopes is not None
+    extended = softcap > 0 or chunk > 0 or sinks is not None or plain_only or kept > 0 or fewer_values or v_dim != head_dim or slopes is not None or distances is not None
     extras = dict(softcap=softcap, chunk=chunk, sinks=sinks, v_head_dim=v_dim, values_in_keys=values_in_keys, value_offset=value_offset,
-                  keep_first=kept, value_heads=value_heads, slopes=slopes) if extended else {}
-    fast_extras = dict(softcap=softcap, chunk=chunk, sinks=sinks, keep_first=kept, value_heads=value_heads, slopes=slopes) if extended else {}
+                  keep_first=kept, value_heads=value_heads, slopes=slopes, distances=distances) if extended else {}
+    fast_extras = dict(softcap=softcap, chunk=chunk, sinks=sinks, keep_first=kept, value_heads=value_heads, slopes=slopes, distances=distances) if extended else {}
+    if key_heads is not None and key_heads != n_kv_heads:
+        fast_extras["key_heads"] = key_heads
     fast_decode = not plain_only and n_dec > 0 and ops.decode_attention_supported(qkv.dtype, n_q_heads, n_kv_heads, head_dim)
     # the MFMA prefill kernel takes positive softmax scales only; anything else runs the plain kernel
-    fast_prefill = (not plain_only and n_dec < n and scale > 0 and not (kept > 0 and (softcap > 0 or slopes is not None))
+    fast_prefill = (not plain_only and n_dec < n and scale > 0 and not (kept > 0 and (softcap > 0 or slopes is not None or distances is not None))
+                    and not (softcap > 0 and distances is not None)
                     and ops.prefill_attention_supported(qkv.dtype, n_q_heads, n_kv_heads, head_dim, k_pages.shape[2]))
-    out = torch.empty((n, n_q_heads * v_dim), dtype=qkv.dtype, device=qkv.device)
+    if "key_heads" in fast_extras and ((n_dec > 0 and not fast_decode) or (n_dec < n and not fast_prefill)):
+        raise ops.KernelError("attention: key pages with fewer heads than key heads are for the sizes that the MFMA kernels take")
+    if out is None:
+        out = torch.empty((n, n_q_heads * v_dim), dtype=qkv.dtype, device=qkv.device)
     # rows with a single new token come first in the batch
     if n_dec > 0:
         if ctx.decode_longest is not None:

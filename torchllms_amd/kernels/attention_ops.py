@@ -40,6 +40,16 @@ def _slopes(slopes: Optional[torch.Tensor], n_q_heads: int) -> Optional[int]:
     return _ptr(slopes)
 
 
+def _distances(table: Optional[torch.Tensor], n_q_heads: int):
+    """``(address, entries per head)`` of a bias by distance given as a table: float32 [query heads, entries], what a
+    (capped) score gains at every distance between key and query (past the table's end: the last entry); None: no bias."""
+    if table is None:
+        return None, 0
+    if not table.is_cuda or table.dtype != torch.float32 or table.dim() != 2 or table.shape[0] != n_q_heads or not table.shape[1] or not table.is_contiguous():
+        raise KernelError(f"attention: distances must be a contiguous float32 GPU matrix of {n_q_heads} rows")
+    return table.data_ptr(), table.shape[1]
+
+
 def _generic_arguments(qkv, n_q_heads, n_kv_heads, head_dim, k_pages, v_pages, token_seq, positions, block_table, out,
                        sinks=None, v_head_dim=None, values_in_keys=False, value_offset=0, keep_first=0, value_heads=None):
     """What both launches of the plain kernel ask of their arguments; returns (tokens, page size, out, value head
@@ -100,6 +110,7 @@ def attention_generic(
     keep_first: int = 0,
     value_heads: Optional[int] = None,
     slopes: Optional[torch.Tensor] = None,
+    distances: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """Attention of each token's query heads (the first Hq * dh columns of ``qkv``) over the paged
     keys and values of its request; returns [n, Hq * dv].  ``softcap`` c > 0: scores become
@@ -110,7 +121,8 @@ def attention_generic(
     ``keep_first`` n > 0: behind a window a query also sees the first n positions of its request.  ``value_heads``:
     the value pages have fewer heads than the key pages, and key head g reads value head ``g % value_heads``
     (several score maps over the same values: the key heads of map m are ``m * value_heads ..``).  ``slopes``: a bias by
-    distance, one 32-bit number per query head that the capped score loses for every position between key and query."""
+    distance, one 32-bit number per query head that the capped score loses for every position between key and query.
+    ``distances`` float32 [Hq, entries], in place of slopes: what the capped score gains by distance, by table."""
     n, page_size, out, v_dim, v_pitch = _generic_arguments(qkv, n_q_heads, n_kv_heads, head_dim, k_pages, v_pages, token_seq,
                                                            positions, block_table, out, sinks, v_head_dim, values_in_keys, value_offset,
                                                            keep_first, value_heads)
@@ -120,7 +132,7 @@ def attention_generic(
             qkv.data_ptr(), qkv.stride(0), out.data_ptr(), out.stride(0), k_pages.data_ptr(), v_at,
             token_seq.data_ptr(), positions.data_ptr(), block_table.data_ptr(), block_table.stride(0), n,
             n_q_heads, n_kv_heads, head_dim, page_size, window, float(scale), float(softcap), int(chunk), _ptr(sinks), v_dim,
-            v_pitch, dtype_code(qkv.dtype), int(keep_first), int(value_heads or 0), _slopes(slopes, n_q_heads), _stream(),
+            v_pitch, dtype_code(qkv.dtype), int(keep_first), int(value_heads or 0), _slopes(slopes, n_q_heads), *_distances(distances, n_q_heads), _stream(),
         )
     )
     return out
@@ -151,6 +163,7 @@ def attention_generic_split(
     keep_first: int = 0,
     value_heads: Optional[int] = None,
     slopes: Optional[torch.Tensor] = None,
+    distances: Optional[torch.Tensor] = None,
 ) -> torch.Tensor:
     """``attention_generic`` for steps with few tokens and long contexts (decode): every block of 64
     keys is computed by a wave of its own and a second kernel joins the blocks in order.  The same
@@ -168,14 +181,15 @@ def attention_generic_split(
             qkv.data_ptr(), qkv.stride(0), out.data_ptr(), out.stride(0), k_pages.data_ptr(), v_at,
             token_seq.data_ptr(), positions.data_ptr(), block_table.data_ptr(), block_table.stride(0), n,
             n_q_heads, n_kv_heads, head_dim, page_size, window, float(scale), float(softcap), int(chunk), _ptr(sinks), v_dim,
-            v_pitch, dtype_code(qkv.dtype), max_blocks, partials.data_ptr(), int(keep_first), int(value_heads or 0), _slopes(slopes, n_q_heads), _stream(),
+            v_pitch, dtype_code(qkv.dtype), max_blocks, partials.data_ptr(), int(keep_first), int(value_heads or 0), _slopes(slopes, n_q_heads),
+            *_distances(distances, n_q_heads), _stream(),
         )
     )
     return out
 
 
 _DECODE_SIGNATURES = {
-    "tl_attn_decode": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P],
+    "tl_attn_decode": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P, _P, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P, _I, _I, _P],
 }
 DECODE_HEAD_DIMS = (32, 64, 128, 256)
 _DECODE_BLOCK_KEYS = 64  # keys one block pass covers (4 waves x 16): splits are multiples of it
@@ -263,10 +277,14 @@ def attention_decode(
     value_heads: Optional[int] = None,
     v_offset: int = 0,
     slopes: Optional[torch.Tensor] = None,
+    distances: Optional[torch.Tensor] = None,
+    key_heads: Optional[int] = None,
 ) -> torch.Tensor:
     """Attention of single-token queries over their requests' pages with the split-KV MFMA kernel.
     ``longest``: an upper bound of any token's visible key range, counted from its 16-aligned first
-    visible key (position + 1 without a window; kept first keys are counted here).  ``softcap``, ``chunk``, ``sinks``, ``slopes``: as ``attention_generic``.
+    visible key (position + 1 without a window; kept first keys are counted here).  ``softcap``, ``chunk``, ``sinks``, ``slopes``, ``distances``: as ``attention_generic``.
+    ``key_heads``: the key pages have fewer heads than ``n_kv_heads``, and key head g reads page head ``g % key_heads`` (more
+    query heads over one key head than a block takes: groups of them as key heads of their own).
     ``keep_first``: behind a window a query also sees that many first positions of its request.  ``value_heads``,
     ``v_offset``: the value pages are [pages, value_heads, page, v_pitch] with ``value_heads`` dividing the kv heads
     (key head g reads value head ``g % value_heads``) and rows of ``v_pitch`` >= dh channels, of which this call takes
@@ -291,7 +309,10 @@ def attention_decode(
     v_pitch = v_pages.shape[3] if v_pages.dim() == 4 else -1
     if keep_first < 0 or v_heads <= 0 or n_kv_heads % v_heads or v_offset < 0 or v_offset + head_dim > v_pitch or v_pitch % 8 or v_offset % 8:
         raise KernelError("attention_decode: kept keys, value heads or the place of the values inside their rows do not fit")
-    if k_pages.dim() != 4 or k_pages.shape[1:] != (n_kv_heads, page_size, head_dim) or k_pages.dtype != qkv.dtype or not k_pages.is_contiguous():
+    k_heads = n_kv_heads if key_heads is None else int(key_heads)
+    if k_heads <= 0 or n_kv_heads % k_heads:
+        raise KernelError(f"attention_decode: {n_kv_heads} key heads are not a multiple of {k_heads} heads of the key pages")
+    if k_pages.dim() != 4 or k_pages.shape[1:] != (k_heads, page_size, head_dim) or k_pages.dtype != qkv.dtype or not k_pages.is_contiguous():
         raise KernelError("attention_decode: key pages must be contiguous [pages, Hkv, page_size, dh] bfloat16")
     if v_pages.dim() != 4 or v_pages.shape[:3] != (k_pages.shape[0], v_heads, page_size) or v_pages.dtype != qkv.dtype or not v_pages.is_contiguous():
         raise KernelError("attention_decode: value pages must be contiguous [pages, value heads, page_size, >= dh] bfloat16")
@@ -316,7 +337,7 @@ def attention_decode(
             token_seq.data_ptr(), positions.data_ptr(), block_table.data_ptr(), block_table.stride(0), n,
             n_q_heads, n_kv_heads, head_dim, page_size, window, float(scale), split_size, n_splits,
             _ptr(ws_o), _ptr(ws_ml), float(softcap), int(chunk), _ptr(sinks), int(keep_first) if (window > 0 or chunk > 0) else 0, v_heads,
-            v_pitch, int(v_offset), v_pitch, int(v_offset), _slopes(slopes, n_q_heads), _stream(),
+            v_pitch, int(v_offset), v_pitch, int(v_offset), _slopes(slopes, n_q_heads), *_distances(distances, n_q_heads), k_heads, _stream(),
         ),
         lib,
         "tl_variant_last_error",
@@ -326,7 +347,7 @@ def attention_decode(
 
 # ----------------------------------------------------------------------------- prefill attention (bfloat16, MFMA)
 _PREFILL_SIGNATURES = {
-    "tl_attn_prefill": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P],
+    "tl_attn_prefill": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _F, _I, _P, _I, _I, _I, _I, _I, _I, _P, _P, _I, _I, _P],
 }
 PREFILL_HEAD_DIMS = (32, 64, 128, 256)
 
@@ -428,10 +449,13 @@ def attention_prefill(
     value_heads: Optional[int] = None,
     v_offset: int = 0,
     slopes: Optional[torch.Tensor] = None,
+    distances: Optional[torch.Tensor] = None,
+    key_heads: Optional[int] = None,
 ) -> torch.Tensor:
     """Causal attention of the rows named by the tile lists (see ``prefill_tiles``) with the MFMA
     prefill kernel.  Token t of ``qkv`` / ``out`` is token t of ``qo_indptr``'s numbering.
-    ``key_groups`` = 2: two sets of waves per block share a tile's keys between them.  ``slopes``: as ``attention_generic``.
+    ``key_groups`` = 2: two sets of waves per block share a tile's keys between them.  ``slopes``, ``distances``: as ``attention_generic``;
+    ``key_heads``: as ``attention_decode``.
     ``keep_first``: behind a window a query also sees that many first positions of its request.  ``value_heads``,
     ``v_offset``: the value pages are [pages, value_heads, page, v_pitch] with ``value_heads`` dividing the kv heads
     (key head g reads value head ``g % value_heads``) and rows of ``v_pitch`` >= dh channels, of which this call takes
@@ -455,7 +479,10 @@ def attention_prefill(
     v_pitch = v_pages.shape[3] if v_pages.dim() == 4 else -1
     if keep_first < 0 or v_heads <= 0 or n_kv_heads % v_heads or v_offset < 0 or v_offset + head_dim > v_pitch or v_pitch % 8 or v_offset % 8:
         raise KernelError("attention_prefill: kept keys, value heads or the place of the values inside their rows do not fit")
-    if k_pages.dim() != 4 or k_pages.shape[1:] != (n_kv_heads, page_size, head_dim) or k_pages.dtype != qkv.dtype or not k_pages.is_contiguous():
+    k_heads = n_kv_heads if key_heads is None else int(key_heads)
+    if k_heads <= 0 or n_kv_heads % k_heads:
+        raise KernelError(f"attention_prefill: {n_kv_heads} key heads are not a multiple of {k_heads} heads of the key pages")
+    if k_pages.dim() != 4 or k_pages.shape[1:] != (k_heads, page_size, head_dim) or k_pages.dtype != qkv.dtype or not k_pages.is_contiguous():
         raise KernelError("attention_prefill: key pages must be contiguous [pages, Hkv, page_size, dh] bfloat16")
     if v_pages.dim() != 4 or v_pages.shape[:3] != (k_pages.shape[0], v_heads, page_size) or v_pages.dtype != qkv.dtype or not v_pages.is_contiguous():
         raise KernelError("attention_prefill: value pages must be contiguous [pages, value heads, page_size, >= dh] bfloat16")
@@ -468,7 +495,7 @@ def attention_prefill(
             qo_indptr.data_ptr(), kv_lens.data_ptr(), block_table.data_ptr(), block_table.stride(0),
             tile_row.data_ptr(), tile_q0.data_ptr(), tile_row.numel(), n_q_heads, n_kv_heads, head_dim, page_size,
             window, float(scale), int(key_groups), float(softcap), int(chunk), _ptr(sinks), int(keep_first), v_heads, v_pitch, int(v_offset),
-            v_pitch, int(v_offset), _slopes(slopes, n_q_heads), _stream(),
+            v_pitch, int(v_offset), _slopes(slopes, n_q_heads), *_distances(distances, n_q_heads), k_heads, _stream(),
         ),
         lib,
         "tl_variant_last_error",

@@ -18,7 +18,6 @@ import shutil
 import subprocess
 import sys
 import tempfile
-import threading
 import time
 from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
@@ -40,8 +39,9 @@ CORE_SOURCES = [
     "routed_ops.hip",
     "stream_ops.hip",
     "retention.hip",
+    "ssd.hip",
 ]
-HEADERS = ["common.h", "qkv_epilogue.h", "no_alloc.h"]
+HEADERS = ["common.h", "qkv_epilogue.h", "no_alloc.h", "recurrence.h"]
 
 HIPCC_FLAGS = [
     f"--offload-arch={ARCH}",
@@ -139,38 +139,27 @@ def build_library(lib_name: str, sources: Sequence[str], defines: Sequence[str] 
     lib = out_dir / f"lib{lib_name}.so"
     _log(f"compiling {lib.name} for {ARCH} from {len(sources)} source file(s) into {out_dir}")
     t0 = time.time()
-    stop = threading.Event()
 
-    def heartbeat():
-        while not stop.wait(20.0):
-            _log(f"... still compiling {lib.name} ({time.time() - t0:.0f} s)")
+    def compile_one(src: str) -> Path:
+        # the process id keeps two processes that build the same library at once (two first calls from
+        # one checkout) out of each other's files; the library itself is moved into place whole
+        obj = out_dir / f"{lib_name}.{Path(src).stem}.{os.getpid()}.o"
+        _run([hipcc, *HIPCC_FLAGS, *defines, "-I", str(CSRC), "-c", str(CSRC / src), "-o", str(obj)], f"compile {src}")
+        _log(f"compiled {src} ({time.time() - t0:.0f} s)")
+        return obj
 
-    beat = threading.Thread(target=heartbeat, daemon=True)
-    beat.start()
-    try:
-        objs = []
-
-        def compile_one(src: str) -> Path:
-            # the process id keeps two processes that build the same library at once (two first calls from
-            # one checkout) out of each other's files; the library itself is moved into place whole
-            obj = out_dir / f"{lib_name}.{Path(src).stem}.{os.getpid()}.o"
-            _run([hipcc, *HIPCC_FLAGS, *defines, "-I", str(CSRC), "-c", str(CSRC / src), "-o", str(obj)], f"compile {src}")
-            return obj
-
-        workers = max(1, min(len(sources), int(os.environ.get("MAX_JOBS", "8")), 16))
-        with ThreadPoolExecutor(max_workers=workers) as pool:
-            objs = list(pool.map(compile_one, sources))
-        tmp = out_dir / f"lib{lib_name}.{os.getpid()}.tmp.so"
-        _run([hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", str(tmp), *map(str, objs)], f"link {lib.name}")
-        os.replace(tmp, lib)
-        lib.with_suffix(".stamp").write_text(digest)
-        for o in objs:
-            try:
-                o.unlink()
-            except OSError:
-                pass
-    finally:
-        stop.set()
+    workers = max(1, min(len(sources), int(os.environ.get("MAX_JOBS", "8")), 16))
+    with ThreadPoolExecutor(max_workers=workers) as pool:
+        objs = list(pool.map(compile_one, sources))
+    tmp = out_dir / f"lib{lib_name}.{os.getpid()}.tmp.so"
+    _run([hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", str(tmp), *map(str, objs)], f"link {lib.name}")
+    os.replace(tmp, lib)
+    lib.with_suffix(".stamp").write_text(digest)
+    for o in objs:
+        try:
+            o.unlink()
+        except OSError:
+            pass
     _log(f"built {lib.name} in {time.time() - t0:.1f} s")
     return lib
 

@@ -10,7 +10,7 @@ from typing import Optional
 
 import torch
 
-from .base import KernelError, _gpu, _i32, _ptr, _stream, check, core, dtype_code
+from .base import F32, KernelError, SplitSums, _gpu, _i32, _ptr, _stream, check, core, dtype_code
 
 #: the widest head ``head_prepare`` takes (sixteen channels a lane)
 HEAD_PREPARE_MAX_DIM = 1024
@@ -118,6 +118,34 @@ def branch_norm_add(stream: torch.Tensor, y: torch.Tensor, weight: torch.Tensor,
     if not want_rows:
         return None
     return stream if y.dtype == torch.float32 else rows
+
+
+def add_norm(stream: torch.Tensor, branch, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,
+             rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``h = stream + branch`` in 32-bit, and ``h / sqrt(mean(h^2) + eps) * weight`` row by row in ``out_dtype``, rounded once.
+    ``stream`` float32 [n, hidden] becomes h in place; with ``rows`` (int32 indices) the result is that of those rows only
+    and the stream stays as it is.  ``branch``: a tensor (float32, or of ``out_dtype``) or a ``SplitSums``, whose slices are
+    added in 32-bit on the way."""
+    partial = branch.partial if isinstance(branch, SplitSums) else None
+    tensor = None if partial is not None else branch
+    _gpu(stream, tensor, partial, weight, rows)
+    _i32(rows, "rows")
+    if stream.dim() != 2 or stream.dtype != torch.float32 or not stream.is_contiguous():
+        raise KernelError("add_norm: the stream must be a contiguous float32 [rows, hidden] tensor")
+    n, hidden = stream.shape
+    if tuple(branch.shape) != (n, hidden) or (tensor is not None and not tensor.is_contiguous()):
+        raise KernelError("add_norm: the branch must have the stream's shape")
+    if partial is not None and (partial.dtype != torch.float32 or partial.stride(2) != 1 or partial.stride(1) != hidden):
+        raise KernelError("add_norm: the slices of the branch must be float32 with rows side by side")
+    if tensor is not None and tensor.dtype not in (torch.float32, out_dtype):
+        raise KernelError(f"add_norm: a branch of {tensor.dtype} with results of {out_dtype}")
+    _f32_vector(weight, hidden, "add_norm: weight")
+    y = torch.empty((n if rows is None else rows.numel(), hidden), dtype=out_dtype, device=stream.device)
+    check(core().tl_add_norm(
+        stream.data_ptr(), _ptr(tensor), F32 if tensor is None else dtype_code(tensor.dtype), _ptr(partial),
+        0 if partial is None else partial.shape[0], 0 if partial is None else partial.stride(0), _ptr(rows), weight.data_ptr(), float(eps),
+        y.data_ptr(), y.shape[0], hidden, dtype_code(out_dtype), _stream()))
+    return y
 
 
 def rmsnorm_columns(x: torch.Tensor, weight: torch.Tensor, eps: float, out_dtype: torch.dtype,

@@ -32,9 +32,9 @@ _CORE_SIGNATURES = {
     "tl_rope_kv_write": [_P, _I, _I, _I, _I, _P, _P, _P, _I, _I, _P, _P, _P, _I, _I, _P],
     "tl_silu_mul": [_P, _P, _I, _I, _I, _P],
     "tl_add_bias": [_P, _P, _I, _I, _I, _I, _P],
-    "tl_attention_generic": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _P, _I, _I, _I, _I, _I, _P, _P],
-    "tl_attention_generic_split": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _P, _I, _I, _I, _I, _P, _I, _I, _P, _P],
-    "tl_embed_scaled": [_P, _P, _P, _I, _I, _F, _I, _P],
+    "tl_attention_generic": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P],
+    "tl_attention_generic_split": [_P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _F, _I, _P, _I, _I, _I, _I, _P, _I, _I, _P, _P, _I, _P],
+    "tl_embed_scaled": [_P, _P, _P, _I, _I, _F, _I, _P, _P, _P],
     "tl_layernorm": [_P, _P, _P, _F, _P, _P, _P, _P, _P, _I, _I, _F, _I, _I, _P],
     "tl_gelu_mul": [_P, _P, _I, _I, _I, _P],
     "tl_rope_norm_kv_write": [_P, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P, _P, _P, _I, _I, _P],
@@ -42,19 +42,27 @@ _CORE_SIGNATURES = {
     "tl_selective_scan": [_P, _P, _I, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P, _I64, _P, _P, _P, _I, _I, _I, _I, _P, _P, _I, _P, _P, _P],
     "tl_gated_delta": [_P, _I, _P, _I, _I, _I, _I, _P, _P, _P, _F, _P, _I64, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _I, _P, _I, _I, _P, _I, _F, _P],
     "tl_matrix_memory": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _I, _P, _F, _P, _I64, _P, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P],
-    "tl_router_topk": [_P, _I, _P, _I, _I, _I, _P, _P, _I, _I, _I, _F, _P, _P],
+    "tl_router_topk": [_P, _I, _P, _I, _I, _I, _P, _P, _I, _I, _I, _F, _P, _I, _P],
     "tl_streams_update": [_P, _I, _I64, _I, _I, _P, _I, _P, _P, _P, _P, _P, _P, _P, _P, _I, _P],
     "tl_streams_open": [_P, _P, _I, _I64, _P],
     "tl_maps_join": [_P, _I, _P, _I, _I, _I, _F, _F, _F, _I, _P],
     "tl_expert_glu_rows": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     "tl_expert_down_rows": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
-    "tl_expert_gather": [_P, _P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
+    "tl_expert_gather": [_P, _P, _P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
+    "tl_pair_rows": [_P, _P, _P, _I, _I, _I, _I, _P],
     "tl_expert_combine": [_P, _I, _P, _P, _P, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _P],
     "tl_bias_gelu": [_P, _P, _I, _I, _I, _P],
     "tl_weighted_pair": [_P, _F, _P, _F, _P, _I64, _I, _P],
     "tl_post_norm_add_norm": [_P, _P, _P, _F, _P, _F, _P, _P, _I, _I, _I, _P],
     "tl_pair_norm_add_norm": [_P, _P, _P, _F, _F, _P, _P, _F, _F, _P, _F, _P, _F, _P, _P, _I, _I, _I, _P],
     "tl_relu_square": [_P, _I64, _I, _P],
+    "tl_add_norm": [_P, _P, _I, _P, _I, _I64, _P, _P, _F, _P, _I, _I, _I, _P],
+    "tl_limited_gate_mul": [_P, _P, _I, _I, _F, _F, _I, _P],
+    "tl_ssd": [_P, _I, _P, _I, _P, _P, _P, _P, _I64, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
+    "tl_ssd_chunks": [_P, _I, _P, _I, _P, _P, _P, _P, _I64, _P, _P, _I, _I, _I, _I, _I, _P, _P, _I, _P, _P, _I, _P],
+    "tl_ssd_segment": [],
+    "tl_ssd_chunk_channels": [],
+    "tl_gated_norm": [_P, _P, _I, _P, _P, _I, _I, _I, _F, _I, _P],
     "tl_retention": [_P, _I, _I, _I, _I, _I, _P, _I, _P, _P, _I64, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P],
     "tl_retention_block_columns": [],
     "tl_retention_chunks": [_P, _I, _I, _I, _I, _I, _P, _I, _P, _P, _I64, _P, _P, _I, _I, _I, _I, _F, _P, _P, _I, _P, _I, _P],
@@ -71,7 +79,7 @@ _CORE_SIGNATURES = {
     "tl_gemm_stream": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "tl_gemm_stream_select": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _I64, _I, _P],
     "tl_gemm_stream_glu_select": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _I64, _I, _P],
-    "tl_gemm_stream_glu": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _I, _F, _I, _P],
+    "tl_gemm_stream_glu": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P, _I, _F, _I, _F, _F, _P],
     "tl_gemm_stream_residual": [_P, _I, _P, _I, _P, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     "tl_gemm_stream_qkv": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P, _P, _I, _I, _P, _I, _F, _P],
     "tl_gemm_wide": [_P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P, _P],

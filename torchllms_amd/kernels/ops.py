@@ -18,6 +18,7 @@ a module's own helpers and tables stay in the module.
 ``stream_ops``       several residual streams with their weighted reads and writes, the norm without statistics,
                      the join of differential attention's two maps
 ``retention_ops``    retention (linear attention with a constant decay per head)
+``ssd_ops``          state-space duality (a decay per head and token) and the gated norm by parts behind it
 ``sampling_ops``     the sampling kernel
 """
 
@@ -105,6 +106,7 @@ from .sequence_ops import (  # noqa: F401
     gated_delta,
     gated_linear,
     gelu_mul,
+    limited_gate_mul,
     layernorm,
     matrix_memory,
     matrix_memory_state_size,
@@ -114,6 +116,7 @@ from .sequence_ops import (  # noqa: F401
 )
 from .head_ops import (  # noqa: F401
     HEAD_PREPARE_MAX_DIM,
+    add_norm,
     branch_norm_add,
     head_prepare,
     pack_heads,
@@ -143,6 +146,14 @@ from .retention_ops import (  # noqa: F401
     RETENTION_SEGMENTS_FROM,
     retention,
     retention_segments_supported,
+)
+from .ssd_ops import (  # noqa: F401
+    SSD_MAX_STATE,
+    SSD_SEGMENT,
+    SSD_SEGMENTS_FROM,
+    gated_norm,
+    ssd,
+    ssd_segments_supported,
 )
 from .stream_ops import (  # noqa: F401
     MAX_STREAMS,

@@ -126,8 +126,9 @@ class PendingProduct(Unfinished):
     def dtype(self):
         return self.x.dtype
 
-    def resolve(self) -> torch.Tensor:
-        return gemm_stream(self.x, self.w, self.x.dtype, self.waves)
+    def resolve(self, dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+        """The product, in the inputs' dtype or as the 32-bit sums that it is made of (``dtype`` float32)."""
+        return gemm_stream(self.x, self.w, dtype or self.x.dtype, self.waves)
 
     def added_to(self, h: torch.Tensor, weight: torch.Tensor, eps: float):
         """``(h + x @ w.T, NormedRows of it)`` for a norm with gain ``weight``."""
@@ -283,16 +284,16 @@ def gemm_wide_qkv(
     return out
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "sigmoid_limited": 2}
 
 
 def gemm_stream_glu(x: torch.Tensor, w: torch.Tensor, waves: int = 0, cols: int = 16, norm: Optional[NormedRows] = None,
-                    activation: str = "silu") -> torch.Tensor:
+                    activation: str = "silu", limit: float = 0.0, slope: float = 1.0) -> torch.Tensor:
     """``act(x @ gate.T) * (x @ up.T)`` for at most 16 rows of bfloat16 ``x`` and ``w`` [2F, K] =
     gate rows | up rows, in one pass over ``w``; rounded as ``silu_mul(linear(x, w))``.  ``cols``: 16
     or 8 columns of the result per block (8: a launch shaped like the plain product's).  ``norm``:
     ``NormedRows`` whose ``gained`` rows ``x`` is; the result is then that of the normed rows.
-    ``activation``: "silu" or "gelu_tanh"."""
+    ``activation``: "silu", "gelu_tanh" or "sigmoid_limited" (``limited_gate_mul`` with ``limit`` and ``slope``)."""
     if activation not in GATE_ACTIVATIONS:
         raise KernelError(f"gemm_stream_glu: activation {activation!r} ({sorted(GATE_ACTIVATIONS)})")
     _gpu(x, w)
@@ -307,7 +308,7 @@ def gemm_stream_glu(x: torch.Tensor, w: torch.Tensor, waves: int = 0, cols: int 
     check(
         core().tl_gemm_stream_glu(
             x.data_ptr(), x.stride(0), w.data_ptr(), w.stride(0), out.data_ptr(), out.stride(0), m, n, k, waves, cols, sums, n_sums, eps,
-            GATE_ACTIVATIONS[activation], _stream(),
+            GATE_ACTIVATIONS[activation], float(limit), float(slope), _stream(),
         )
     )
     return out
@@ -648,25 +649,29 @@ def linear_to_sum(x: torch.Tensor, w: torch.Tensor, may_wait: bool = False):
     return run_choice(choice, x, w, x.dtype, leave_split=True)
 
 
-def linear_glu(x: torch.Tensor, w: torch.Tensor, activation: str = "silu") -> torch.Tensor:
+def linear_glu(x: torch.Tensor, w: torch.Tensor, activation: str = "silu", limit: float = 0.0, slope: float = 1.0) -> torch.Tensor:
     """``act(x @ gate.T) * (x @ up.T)`` for ``w`` [2F, K] = gate rows | up rows.  With silu: one fused
     kernel where one of the decode kernels serves the shape, else the product followed by the gate.  ``x``
     may be ``NormedRows``: the weight-streaming kernel applies them, for any other they are normed first.
-    With "gelu_tanh" the weight-streaming kernel (up to 16 rows) takes the gate into itself as well; every other
+    With "gelu_tanh" or "sigmoid_limited" (``g * sigmoid(slope * g) * (u + 1)``, g and u between limits: see
+    ``limited_gate_mul``) the weight-streaming kernel (up to 16 rows) takes the gate into itself as well; every other
     product is followed by the gate's kernel."""
     if activation != "silu":
-        if activation != "gelu_tanh":
-            raise KernelError(f"linear_glu: activation {activation!r} (silu, gelu_tanh)")
-        from .sequence_ops import gelu_mul
+        if activation not in GATE_ACTIVATIONS:
+            raise KernelError(f"linear_glu: activation {activation!r} ({sorted(GATE_ACTIVATIONS)})")
+        from .sequence_ops import gelu_mul, limited_gate_mul
+
+        def gate(both):
+            return gelu_mul(both) if activation == "gelu_tanh" else limited_gate_mul(both, limit, slope)
 
         x = resolved(x)
         if x.dtype == torch.bfloat16:
             _gpu(x, w)
             choice = linear_choice(x, w, "glu")
             if choice is not None and choice[0] == "stream":
-                return gemm_stream_glu(x, w, choice[1], choice[2] if len(choice) > 2 else 16, activation=activation)
-            return gelu_mul(run_choice(choice, x, w, x.dtype))
-        return gelu_mul(linear(x, w))
+                return gemm_stream_glu(x, w, choice[1], choice[2] if len(choice) > 2 else 16, activation=activation, limit=limit, slope=slope)
+            return gate(run_choice(choice, x, w, x.dtype))
+        return gate(linear(x, w))
     if isinstance(x, NormedRows):
         choice = linear_choice(x.gained, w, "glu")
         if choice is not None and choice[0] == "stream":

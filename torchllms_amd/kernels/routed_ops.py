@@ -13,17 +13,22 @@ from .base import F32, KernelError, _gpu, _ptr, _stream, check, core, dtype_code
 
 #: the most outputs a router may have (experts and experts that hand their input through together)
 ROUTER_MAX_OUTPUTS = 512
+ROUTER_SCORES = {"softmax": 0, "sigmoid": 1}
 
 
 def router_topk(z: torch.Tensor, n_out: int, correction: Optional[torch.Tensor], top: int, groups: int = 0, keep_groups: int = 0,
-                normalize: bool = False, scale: float = 1.0, bias: Optional[torch.Tensor] = None) -> Tuple[torch.Tensor, torch.Tensor]:
+                normalize: bool = False, scale: float = 1.0, bias: Optional[torch.Tensor] = None,
+                scores: str = "softmax") -> Tuple[torch.Tensor, torch.Tensor]:
     """``z`` float32 [n, >= n_out]: the router's outputs in the first ``n_out`` columns.  ``s = softmax(z)``; the
     ``top`` outputs with the largest ``s + correction`` are chosen (of equal ones the lower index).  Returns
     ``(ids int32 [n, top], weights float32 [n, top])``, the weights being the chosen outputs' ``s``.  ``correction``
     None: the largest ``s``.  ``groups`` g > 0: the outputs form g equal groups of neighbours, a group's score is the
     largest ``s`` in it, and only outputs of the ``keep_groups`` best groups can be chosen.  ``normalize``: the weights
     are divided by their sum (+ 1e-20); ``scale`` then multiplies them.  ``bias`` (float32 [n_out]) is added to ``z``
-    first; with ``normalize`` the weights are then the softmax of ``z + bias`` over the chosen outputs alone."""
+    first; with ``normalize`` the weights are then the softmax of ``z + bias`` over the chosen outputs alone.
+    ``scores`` "sigmoid": ``s`` is the logistic function of every output by itself instead of the softmax over all."""
+    if scores not in ROUTER_SCORES:
+        raise KernelError(f"router_topk: scores {scores!r} ({sorted(ROUTER_SCORES)})")
     _gpu(z, correction, bias)
     if z.dim() != 2 or z.dtype != torch.float32 or z.stride(1) != 1 or z.shape[1] < n_out:
         raise KernelError(f"router_topk: z must be float32 [n, >= {n_out}] with contiguous rows")
@@ -38,7 +43,7 @@ def router_topk(z: torch.Tensor, n_out: int, correction: Optional[torch.Tensor],
     ids = torch.empty((n, top), dtype=torch.int32, device=z.device)
     weights = torch.empty((n, top), dtype=torch.float32, device=z.device)
     check(core().tl_router_topk(z.data_ptr(), z.stride(0), _ptr(correction), n, n_out, top, ids.data_ptr(), weights.data_ptr(),
-                                int(groups), int(keep_groups), 1 if normalize else 0, float(scale), _ptr(bias), _stream()))
+                                int(groups), int(keep_groups), 1 if normalize else 0, float(scale), _ptr(bias), ROUTER_SCORES[scores], _stream()))
     return ids, weights
 
 
@@ -93,12 +98,14 @@ def expert_down_rows(mid: torch.Tensor, w_down: torch.Tensor, offsets: torch.Ten
 PAIR_PRODUCTS_MOST = 4
 
 
-def expert_pair_products(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
+def expert_pair_products(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor,
+                         input_weights: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``y[t, j] = Wd[e] (silu(Wg[e] x[t]) * (Wu[e] x[t]))`` with ``e = ids[t, j]`` for the few pairs of a small decode
     step, each pair by the weight-streaming products that dense layers use (bfloat16; the gate and up products are
     rounded to bfloat16 before the activation, as theirs are), told on the device which expert's matrix to read.  A
-    pair whose ``e`` is no expert of the weights gets some expert's result, which nobody reads.  Returns float32
-    [n * top, D], the pairs in their own order."""
+    pair whose ``e`` is no expert of the weights gets some expert's result, which nobody reads.  ``input_weights`` float32
+    [n, top]: a pair's expert works on ``input_weights[t, j] * x[t]``.  Returns float32 [n * top, D], the pairs in their
+    own order."""
     _gpu(x, w_gate_up, w_down, ids)
     E = w_gate_up.shape[0] if w_gate_up.dim() == 3 else -1
     _pairs(x, ids, E)
@@ -117,28 +124,41 @@ def expert_pair_products(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch
     mid = torch.empty((pairs, F), dtype=x.dtype, device=x.device)
     y = torch.empty((pairs, D), dtype=torch.float32, device=x.device)
     lib, stream = core(), _stream()
+    rows, share = x, top  # pair p reads row p // share of rows
+    if input_weights is not None:
+        _input_weights(input_weights, n, top)
+        rows, share = torch.empty((pairs, D), dtype=x.dtype, device=x.device), 1
+        check(lib.tl_pair_rows(x.data_ptr(), input_weights.data_ptr(), rows.data_ptr(), n, top, D, dtype_code(x.dtype), stream))
     for p in range(pairs):
         which = ids.data_ptr() + 4 * p
-        check(lib.tl_gemm_stream_glu_select(x.data_ptr() + 2 * D * (p // top), D, w_gate_up.data_ptr(), D, mid.data_ptr() + 2 * F * p, F,
+        check(lib.tl_gemm_stream_glu_select(rows.data_ptr() + 2 * D * (p // share), D, w_gate_up.data_ptr(), D, mid.data_ptr() + 2 * F * p, F,
                                             1, F, D, 0, 16, which, 2 * F * D, E, stream))
         check(lib.tl_gemm_stream_select(mid.data_ptr() + 2 * F * p, F, w_down.data_ptr(), F, y.data_ptr() + 4 * D * p, D, 1, D, F,
                                         F32, 0, which, D * F, E, stream))
     return y
 
 
-def expert_gather(x: torch.Tensor, ids: torch.Tensor, n_out: int):
+def _input_weights(weights: torch.Tensor, n: int, top: int) -> None:
+    if tuple(weights.shape) != (n, top) or weights.dtype != torch.float32 or not weights.is_contiguous() or not weights.is_cuda:
+        raise KernelError(f"routed experts: weights of the experts' inputs must be contiguous float32 [{n}, {top}] on the GPU")
+
+
+def expert_gather(x: torch.Tensor, ids: torch.Tensor, n_out: int, input_weights: Optional[torch.Tensor] = None):
     """The (token, choice) pairs in the order of their experts.  Returns ``(rows, pos, offsets)``: ``rows`` [n * top, D]
     holds for every pair its token's row of ``x``, the pairs of output e in the rows ``offsets[e] .. offsets[e + 1]``
-    (int32 [n_out + 1], on the device); ``pos`` int32 [n, top] says which row each pair got."""
+    (int32 [n_out + 1], on the device); ``pos`` int32 [n, top] says which row each pair got.  ``input_weights`` float32
+    [n, top]: a pair's row is its token's row times its weight, rounded."""
     _gpu(x, ids)
     _pairs(x, ids, 0)
     n, D = x.shape
     top = ids.shape[1]
+    if input_weights is not None:
+        _input_weights(input_weights, n, top)
     work = torch.zeros(3 * n_out + 1, dtype=torch.int32, device=x.device)
     counts, offsets, cursor = work[:n_out], work[n_out : 2 * n_out + 1], work[2 * n_out + 1 :]
     pos = torch.empty((n, top), dtype=torch.int32, device=x.device)
     rows = torch.empty((n * top, D), dtype=x.dtype, device=x.device)
-    check(core().tl_expert_gather(x.data_ptr(), ids.data_ptr(), n, top, n_out, counts.data_ptr(), offsets.data_ptr(), cursor.data_ptr(),
+    check(core().tl_expert_gather(x.data_ptr(), ids.data_ptr(), _ptr(input_weights), n, top, n_out, counts.data_ptr(), offsets.data_ptr(), cursor.data_ptr(),
                                   pos.data_ptr(), rows.data_ptr(), D, dtype_code(x.dtype), _stream()))
     return rows, pos, offsets
 
@@ -147,7 +167,7 @@ def expert_combine(
     y: torch.Tensor,
     pos: torch.Tensor,
     ids: torch.Tensor,
-    weights: torch.Tensor,
+    weights: Optional[torch.Tensor],
     n_experts: int,
     x: torch.Tensor,
     shared: Optional[torch.Tensor] = None,
@@ -155,7 +175,7 @@ def expert_combine(
 ) -> torch.Tensor:
     """``out[t] = sum_j weights[t, j] * (y[pos[t, j]] if ids[t, j] < n_experts else x[t])``, plus
     ``sigmoid(shared_gate[t]) * shared[t]`` (``shared[t]`` as it is without a gate): the experts' results (rows in the order ``expert_gather`` gave them) back
-    in the order of the tokens; ``y`` is 32-bit (``expert_down_rows``) or of x's dtype (matrix products over the
+    in the order of the tokens (``weights`` None: added as they are); ``y`` is 32-bit (``expert_down_rows``) or of x's dtype (matrix products over the
     gathered rows).  Returns [n, D] of x's dtype."""
     _gpu(y, pos, ids, weights, x, shared, shared_gate)
     _pairs(x, ids, n_experts)
@@ -165,7 +185,7 @@ def expert_combine(
         raise KernelError("expert_combine: y must be a contiguous [rows, D] matrix of x's dtype or of float32")
     if tuple(pos.shape) != (n, top) or pos.dtype != torch.int32 or not pos.is_contiguous():
         raise KernelError("expert_combine: pos must be contiguous int32 [n, top]")
-    if tuple(weights.shape) != (n, top) or weights.dtype != torch.float32 or not weights.is_contiguous():
+    if weights is not None and (tuple(weights.shape) != (n, top) or weights.dtype != torch.float32 or not weights.is_contiguous()):
         raise KernelError("expert_combine: weights must be contiguous float32 [n, top]")
     sg_stride = 0
     if shared is not None:
@@ -175,7 +195,7 @@ def expert_combine(
             raise KernelError("expert_combine: the shared expert's gate must be float32, one number a token")
         sg_stride = shared_gate.stride(0) if (n > 1 and shared_gate is not None) else 1
     out = torch.empty((n, D), dtype=x.dtype, device=x.device)
-    check(core().tl_expert_combine(y.data_ptr(), 1 if y.dtype == torch.float32 else 0, pos.data_ptr(), ids.data_ptr(), weights.data_ptr(), top, n_experts, x.data_ptr(),
+    check(core().tl_expert_combine(y.data_ptr(), 1 if y.dtype == torch.float32 else 0, pos.data_ptr(), ids.data_ptr(), _ptr(weights), top, n_experts, x.data_ptr(),
                                    _ptr(shared), _ptr(shared_gate), sg_stride, out.data_ptr(), n, D, dtype_code(x.dtype), _stream()))
     return out
 

@@ -34,16 +34,25 @@ class ScaledSum(Unfinished):
         return (total * self.mult).to(self.terms[0].dtype)
 
 
-def embed_scaled(tokens: torch.Tensor, table: torch.Tensor, scale: float) -> torch.Tensor:
-    """``float(table[tokens]) * scale`` as a 32-bit tensor [n, hidden]."""
-    _gpu(tokens, table)
+def embed_scaled(tokens: torch.Tensor, table: torch.Tensor, scale: float, positions: Optional[torch.Tensor] = None,
+                 position_table: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``float(table[tokens]) * scale`` as a 32-bit tensor [n, hidden]; with ``position_table`` [positions, hidden] (of the
+    table's dtype) plus ``float(position_table[positions])``.  The caller has checked that tokens and positions lie in
+    their tables."""
+    _gpu(tokens, table, positions, position_table)
     _i32(tokens, "tokens")
+    _i32(positions, "positions")
+    if position_table is not None:
+        if position_table.dim() != 2 or position_table.shape[1] != table.shape[-1] or position_table.dtype != table.dtype or not position_table.is_contiguous():
+            raise KernelError("embedding: position vectors must be a contiguous matrix of the table's width and dtype")
+        if positions is None or positions.numel() != tokens.numel():
+            raise KernelError("embedding: position vectors need one position per token")
     if table.dim() != 2 or not table.is_contiguous():
         raise KernelError("embedding table must be a contiguous matrix")
     n, hidden = tokens.numel(), table.shape[1]
     out = torch.empty((n, hidden), dtype=torch.float32, device=table.device)
     check(core().tl_embed_scaled(tokens.data_ptr(), table.data_ptr(), out.data_ptr(), n, hidden, float(scale),
-                                 dtype_code(table.dtype), _stream()))
+                                 dtype_code(table.dtype), _ptr(positions), _ptr(position_table), _stream()))
     return out
 
 
@@ -101,6 +110,18 @@ def gelu_mul(gate_up: torch.Tensor) -> torch.Tensor:
     n, inter = gate_up.shape[0], gate_up.shape[1] // 2
     out = torch.empty((n, inter), dtype=gate_up.dtype, device=gate_up.device)
     check(core().tl_gelu_mul(gate_up.data_ptr(), out.data_ptr(), n, inter, dtype_code(gate_up.dtype), _stream()))
+    return out
+
+
+def limited_gate_mul(gate_up: torch.Tensor, limit: float, slope: float) -> torch.Tensor:
+    """``g * sigmoid(slope * g) * (u + 1)`` with ``g = min(gate, limit)`` and ``u`` the up half between -limit and limit, for
+    ``gate_up`` [n, 2F] = gate | up, computed in 32-bit, rounded once."""
+    _gpu(gate_up)
+    if gate_up.dim() != 2 or gate_up.shape[1] % 2 or not gate_up.is_contiguous():
+        raise KernelError("limited_gate_mul input must be contiguous [n, 2F]")
+    n, inter = gate_up.shape[0], gate_up.shape[1] // 2
+    out = torch.empty((n, inter), dtype=gate_up.dtype, device=gate_up.device)
+    check(core().tl_limited_gate_mul(gate_up.data_ptr(), out.data_ptr(), n, inter, float(limit), float(slope), dtype_code(gate_up.dtype), _stream()))
     return out
 
 

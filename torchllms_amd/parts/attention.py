@@ -11,7 +11,7 @@ from ..config.spec import PartSpec
 from ..kernels import ops
 from ..kernels.attention import paged_attention
 from .base import MIXERS, POSITIONS, KVNeed, Mixer, ParamSpec, StateNeed
-from .positions import step_table
+from .positions import distance_bucket_starts, distance_table, step_table
 
 
 #: (heads, kv heads, head size) whose fall to the plain attention kernel has been reported
@@ -51,7 +51,9 @@ class Attention(Mixer):
     positions; their pages are never given back.
 
     ``slopes``: a bias by distance: one number per query head, and head h's (capped) score loses ``slopes[h] * (i - j)``
-    between the query at position i and the key at position j.
+    between the query at position i and the key at position j.  ``distance_rows`` B > 0 (with ``distance_most``): a learned
+    bias by bucketed distance instead (tensor ``distances`` [B, num_heads], unscaled): the (capped) score gains
+    ``distances[bucket(i - j), h]``, a bucket a distance below B / 2 and then logarithmic ones up to ``distance_most``.
     """
 
     #: every launch is fixed by the step's shape: a decode step may be recorded in a HIP graph
@@ -84,6 +86,8 @@ class Attention(Mixer):
         values_from_keys: bool = False,
         keep_first: int = 0,
         slopes: Optional[Sequence[float]] = None,
+        distance_rows: int = 0,
+        distance_most: int = 0,
     ):
         self.values_from_keys = bool(values_from_keys)
         self.keep_first = int(keep_first)
@@ -113,6 +117,12 @@ class Attention(Mixer):
             raise ValueError(f"attention: {len(slopes)} slopes for {num_heads} heads")
         self.slope_values = None if slopes is None else [float(v) for v in slopes]
         self.slopes: Optional[torch.Tensor] = None
+        self.distance_rows, self.distance_most = int(distance_rows), int(distance_most)
+        if self.distance_rows and slopes is not None:
+            raise ValueError("attention: slopes and a table of distances are one bias by distance each")
+        if self.distance_rows:
+            distance_bucket_starts(self.distance_rows, self.distance_most)  # (refuses what has no buckets)
+        self.distances: Optional[torch.Tensor] = None
         self.qk_norm_weight = bool(qk_norm_weight)
         self.q_temp_coef = float(q_temp_coef)
         self.q_temp_every = int(q_temp_every)
@@ -151,7 +161,7 @@ class Attention(Mixer):
     def extended(self) -> bool:
         """Whether the layer needs what only the unfused path and the plain attention kernel do."""
         return (self.v_head_dim != self.head_dim or self.qk_norm_eps > 0 or self.softcap > 0 or self.chunk > 0 or self.has_sinks
-                or self.slope_values is not None)
+                or self.slope_values is not None or self.distance_rows > 0)
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         q = self.num_heads * self.head_dim
@@ -164,6 +174,8 @@ class Attention(Mixer):
                 specs["wv.weight"] = ParamSpec((self.num_kv_heads * self.v_head_dim, self.hidden_size))
         if self.has_sinks:
             specs["sinks"] = ParamSpec((self.num_heads,), kind="vector", init="zeros")
+        if self.distance_rows:
+            specs["distances"] = ParamSpec((self.distance_rows, self.num_heads), kind="vector")
         if self.qkv_bias:
             specs["wq.bias"] = ParamSpec((q,), init="zeros")
             if not self.shares_kv:
@@ -230,6 +242,8 @@ class Attention(Mixer):
             self.sinks = tensors["sinks"].float().contiguous()
         if self.slope_values is not None:
             self.slopes = torch.tensor(self.slope_values, dtype=torch.float64).float().to(self.wo.device)
+        if self.distance_rows:
+            self.distances = distance_table(tensors["distances"], self.distance_most, self.window)
         self.position.to(self.wo.device)
 
     def linear_weights(self):
@@ -287,7 +301,7 @@ class Attention(Mixer):
         attn = paged_attention(
             qkv, self.num_heads, self.num_kv_heads, self.head_dim, cache.k_pages, cache.v_pages, ctx, g, self.window,
             self.softmax_scale, softcap=self.softcap, chunk=self.chunk, sinks=self.sinks, v_head_dim=self.v_head_dim,
-            keep_first=self.keep_first, slopes=self.slopes,
+            keep_first=self.keep_first, slopes=self.slopes, distances=self.distances,
         )
         return ops.linear_to_sum(attn, self.wo, may_wait=True)
 
@@ -304,8 +318,10 @@ class Attention(Mixer):
             v_first = ctx.scratch.get(("value_mix", self.value_mix_key))
             if v_first is None:
                 raise RuntimeError(f"attention: no earlier layer of this step has left values under {self.value_mix_key!r}")
+        # queries that nothing prepares stay where they are, and the keys and values alone go to their pages
+        n_q = H if self.bqkv is not None or self.qk_norm_weight or table is not None or self.q_temp_coef != 0.0 or not store else 0
         ops.head_prepare(
-            rows, H, n_kv_in_row, dk, dv if n_kv_in_row else 0, bias=self.bqkv,
+            rows if n_q else rows[:, H * dk :], n_q, n_kv_in_row, dk, dv if n_kv_in_row else 0, bias=self.bqkv,
             q_norm=self.q_norm, k_norm=self.k_norm if n_kv_in_row else None, norm_dims=dk if self.qk_norm_weight else 0,
             eps=self.qk_norm_eps, cos_sin=table, rot_offset=0, rot_dims=rot.rotary_dim if rot else 0,
             pairing=rot.pairing if rot else 0, positions=ctx.positions, temp_coef=self.q_temp_coef, temp_every=self.q_temp_every,
@@ -318,7 +334,7 @@ class Attention(Mixer):
         attn = paged_attention(
             rows, H, self.num_kv_heads, dk, cache.k_pages, cache.v_pages, ctx, g, self.window, self.softmax_scale,
             softcap=self.softcap, chunk=self.chunk, sinks=self.sinks, v_head_dim=dv, keep_first=self.keep_first,
-            slopes=self.slopes,
+            slopes=self.slopes, distances=self.distances,
         )
         if self.out_gate is not None:
             gate_at = v_at + n_kv_in_row * dv

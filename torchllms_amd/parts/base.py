@@ -282,6 +282,11 @@ class Embedding(Part):
         """int32 token ids [n] -> [n, hidden]."""
         raise NotImplementedError
 
+    def forward_at(self, tokens: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+        """``forward`` of tokens at their positions (int32 [n]): what a model calls.  An embedding that knows positions
+        overrides it."""
+        return self.forward(tokens)
+
 
 class Head(Part):
     def forward(self, x: torch.Tensor) -> torch.Tensor:

@@ -27,6 +27,18 @@ class PreNormBlock(Block):
         return h, f
 
 
+@BLOCKS.register("pre_norm_mixer")
+class PreNormMixerBlock(Block):
+    """The same layer without a feed-forward: ``out = x + mixer(norm(x))``."""
+
+    graph_safe = True
+    SLOTS = {"mixer_norm": "norm", "mixer": "mixer"}
+
+    def forward(self, h, delta, ctx, cache):
+        h, y = self.mixer_norm.forward_add_for(self.mixer, h, delta)
+        return h, self.mixer.forward(y, ctx, cache["mixer"])
+
+
 class _Parallel(Block):
     """One norm whose output every branch of the layer reads: ``x <- x + mult * (sum of the branches)``.
     The sum is handed on unapplied (``ops.ScaledSum``), so that the next norm's kernel adds it."""

@@ -14,28 +14,44 @@ from .base import EMBEDDINGS, HEADS, Embedding, Head, ParamSpec
 class TokenEmbedding(Embedding):
     """``h = weight[token]`` (reference: torchllms/models/networks.py:793,1017, which has no scale
     factor).  ``stream_dtype`` "float32": the rows open a 32-bit residual stream whatever the model's
-    dtype, as ``float(weight[token]) * scale``."""
+    dtype, as ``float(weight[token]) * scale``; ``positions`` n > 0: plus a learned vector of the token's position, unscaled
+    (tensor ``positions`` [n, hidden]; beside the 32-bit stream only)."""
 
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, stream_dtype: Optional[str] = None):
+    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, stream_dtype: Optional[str] = None, positions: int = 0):
         if stream_dtype not in (None, "float32"):
             raise ValueError(f"embedding: stream_dtype {stream_dtype!r} (None: the model's dtype, or \"float32\")")
-        if stream_dtype is None and float(scale) != 1.0:
-            raise ValueError("embedding: a scale factor needs the 32-bit residual stream (stream_dtype=\"float32\")")
+        if stream_dtype is None and (float(scale) != 1.0 or positions):
+            raise ValueError("embedding: a scale factor or position vectors need the 32-bit residual stream (stream_dtype=\"float32\")")
+        if positions < 0:
+            raise ValueError(f"embedding: {positions} position vectors")
         self.vocab_size = vocab_size
         self.hidden_size = hidden_size
         self.scale = float(scale)
         self.stream_dtype = stream_dtype
+        self.n_positions = int(positions)
         self.weight: Optional[torch.Tensor] = None
+        self.positions: Optional[torch.Tensor] = None
 
     def param_specs(self) -> Dict[str, ParamSpec]:
-        return {"weight": ParamSpec((self.vocab_size, self.hidden_size))}
+        specs = {"weight": ParamSpec((self.vocab_size, self.hidden_size))}
+        if self.n_positions:
+            specs["positions"] = ParamSpec((self.n_positions, self.hidden_size))
+        return specs
 
     def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
         self.weight = tensors["weight"].contiguous()
+        self.positions = tensors["positions"].contiguous() if self.n_positions else None
+
+    def forward_at(self, tokens: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+        if self.positions is None:
+            return self.forward(tokens)
+        return ops.embed_scaled(tokens, self.weight, self.scale, positions, self.positions)
 
     def forward(self, tokens: torch.Tensor) -> torch.Tensor:
+        if self.positions is not None:
+            raise ValueError("embedding: a token's row depends on its position here (forward_at)")
         if self.stream_dtype == "float32":
             return ops.embed_scaled(tokens, self.weight, self.scale)
         return ops.embed(tokens, self.weight)

@@ -13,14 +13,19 @@ from .base import FEED_FORWARDS, FeedForward, ParamSpec
 @FEED_FORWARDS.register("swiglu")
 class SwiGLU(FeedForward):
     """``w2( act(w1 x) * (w3 x) )`` without biases, act = silu
-    (reference: torchllms/models/networks.py:592-605) or, with ``activation="gelu_tanh"``, the tanh form of gelu."""
+    (reference: torchllms/models/networks.py:592-605) or, with ``activation="gelu_tanh"``, the tanh form of gelu.
+    ``activation="sigmoid_limited"`` (with ``limit`` and ``slope``): ``w2( g sigmoid(slope g) * (u + 1) )`` with g = w1 x kept below
+    ``limit`` and u = w3 x between -limit and limit."""
 
     graph_safe = True
     takes_normed_rows = True
 
-    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu"):
-        if activation not in ("silu", "gelu_tanh"):
-            raise ValueError(f"gated feed-forward: activation {activation!r} (silu, gelu_tanh)")
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "silu", limit: float = 0.0, slope: float = 1.0):
+        if activation not in ("silu", "gelu_tanh", "sigmoid_limited"):
+            raise ValueError(f"gated feed-forward: activation {activation!r} (silu, gelu_tanh, sigmoid_limited)")
+        if activation == "sigmoid_limited" and not limit > 0:
+            raise ValueError(f"gated feed-forward: limit must be positive, got {limit!r}")
+        self.limit, self.slope = float(limit), float(slope)
         self.activation = activation
         self.hidden_size = hidden_size
         self.intermediate_size = intermediate_size
@@ -40,7 +45,7 @@ class SwiGLU(FeedForward):
         return [(self.w13, "glu"), (self.w2, "sum")]
 
     def forward(self, x, ctx):
-        return ops.linear_to_sum(ops.linear_glu(x, self.w13, self.activation), self.w2, may_wait=True)
+        return ops.linear_to_sum(ops.linear_glu(x, self.w13, self.activation, self.limit, self.slope), self.w2, may_wait=True)
 
 
 @FEED_FORWARDS.register("dense_gelu")
@@ -106,7 +111,9 @@ class RoutedExperts(FeedForward):
     the experts form g equal groups of neighbours, a group's score is the largest score in it, and only experts of
     the best ``keep_groups`` groups can be chosen.  ``normalize``: the chosen scores are divided by their sum
     (+ 1e-20); ``route_scale`` then multiplies them.  ``router_bias``: a vector (tensor ``router.bias``) is added to the
-    router's outputs; with ``normalize`` the weights are the softmax of the chosen outputs alone.
+    router's outputs; with ``normalize`` the weights are the softmax of the chosen outputs alone.  ``scores`` "sigmoid": the
+    scores are the logistic function of every output by itself.  ``weigh`` "input": a weight multiplies what its expert
+    works on instead of what comes out.
 
     A token's result depends on nothing but the token.  The (token, choice) pairs of a step are put in the order of
     their experts on the device, and a kernel walks every expert's rows with the expert's weights read once for eight
@@ -123,7 +130,7 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden_size: int, expert_size: int, num_experts: int, top: int, num_identity: int = 0, shared_size: int = 0,
                  shared_gate: bool = True, correction: bool = True, groups: int = 0, keep_groups: int = 0, normalize: bool = False,
-                 route_scale: float = 1.0, router_bias: bool = False):
+                 route_scale: float = 1.0, router_bias: bool = False, scores: str = "softmax", weigh: str = "output"):
         for name, v in (("expert_size", expert_size), ("num_experts", num_experts), ("top", top)):
             if not isinstance(v, int) or v <= 0:
                 raise ValueError(f"routed: {name} must be a positive integer, got {v!r}")
@@ -131,6 +138,11 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"routed: {top} choices among {num_experts} + {num_identity} outputs; sizes must not be negative")
         self.hidden_size, self.F, self.E, self.I, self.top, self.shared = hidden_size, expert_size, num_experts, num_identity, top, shared_size
         self.shared_gate, self.has_correction = bool(shared_gate) and shared_size > 0, bool(correction)
+        if scores not in ("softmax", "sigmoid") or weigh not in ("output", "input"):
+            raise ValueError("routed: scores is \"softmax\" or \"sigmoid\", weigh \"output\" or \"input\"")
+        if weigh == "input" and num_identity:
+            raise ValueError("routed: experts that hand their input through are weighed behind")
+        self.scores, self.weigh_input = scores, weigh == "input"
         self.has_router_bias, self.router_bias = bool(router_bias), None
         self.groups, self.keep_groups, self.normalize, self.route_scale = int(groups or 0), int(keep_groups or 0), bool(normalize), float(route_scale)
         n_out = num_experts + num_identity
@@ -196,7 +208,10 @@ class RoutedExperts(FeedForward):
         n_out = self.E + self.I
         z = ops.linear(x, self.w_router, out_dtype=torch.float32)
         ids, weights = ops.router_topk(z, n_out, self.correction, self.top, groups=self.groups, keep_groups=self.keep_groups,
-                                       normalize=self.normalize, scale=self.route_scale, bias=self.router_bias)
+                                       normalize=self.normalize, scale=self.route_scale, bias=self.router_bias, scores=self.scores)
+        inputs = None  # weights of the experts' inputs; the results are then added as they are
+        if self.weigh_input:
+            inputs, weights = weights, None
         shared = gate = None
         if self.shared:
             shared = ops.linear(ops.linear_glu(x, self.shared_w13), self.shared_w2)
@@ -204,9 +219,9 @@ class RoutedExperts(FeedForward):
         pairs = x.shape[0] * self.top
         if x.dtype == torch.bfloat16 and pairs <= ops.PAIR_PRODUCTS_MOST and self.hidden_size % 8 == 0 and self.F % 8 == 0:
             # a decode step of one or two requests: every pair by the dense layers' weight-streaming products
-            y = ops.expert_pair_products(x, self.w_gu, self.w_down, ids)
+            y = ops.expert_pair_products(x, self.w_gu, self.w_down, ids, input_weights=inputs)
             return ops.expert_combine(y, self._own_rows(x.shape[0], x.device), ids, weights, self.E, x, shared, gate)
-        rows, pos, offsets = ops.expert_gather(x, ids, n_out)
+        rows, pos, offsets = ops.expert_gather(x, ids, n_out, input_weights=inputs)
         if x.dtype == torch.float32 or ctx.host.max_q_len <= 1 or x.shape[0] * self.top < self.GROUPED_FROM:
             y = ops.expert_down_rows(ops.expert_glu_rows(rows, self.w_gu, offsets), self.w_down, offsets)
             return ops.expert_combine(y, pos, ids, weights, self.E, x, shared, gate)

@@ -181,7 +181,7 @@ class Model:
 
     def forward(self, ctx, cache) -> torch.Tensor:
         """Run this step's tokens; returns float32 logits [len(ctx.logit_rows), vocab]."""
-        h = self.embedding.forward(ctx.tokens)
+        h = self.embedding.forward_at(ctx.tokens, ctx.positions)
         delta = None
         order = self.spec.order
         if order:

@@ -24,7 +24,8 @@ class RMSNorm(Norm):
     ``c + weight``) and a second vector may follow it (``scaled``: the tensor ``scale``, a layer's scale on a normed
     branch): ``y = x32 * rsqrt(mean(x32^2) + eps) * (c + weight32) * scale32``.  Both are folded into one 32-bit
     vector when the tensors arrive (``factor``).  ``forward_branch_then`` adds a normed branch to the stream and
-    hands on what another norm makes of the new stream, in one pass."""
+    hands on what another norm makes of the new stream, in one pass.  ``forward_add`` adds a branch to the stream in place
+    (split products as they are, in 32-bit) and norms the sum, in one pass too."""
 
     graph_safe = True
     takes_split_sums = True  # ops.rmsnorm adds the slices of a split product while it reads them
@@ -39,7 +40,6 @@ class RMSNorm(Norm):
         self.stream_dtype = stream_dtype
         self.offset = float(offset)
         self.scaled = bool(scaled)
-        self.takes_split_sums = stream_dtype is None
         self.weight: Optional[torch.Tensor] = None
         self.out_dtype: Optional[torch.dtype] = None
 
@@ -105,11 +105,17 @@ class RMSNorm(Norm):
             raise ValueError("rmsnorm: forward_branch needs the 32-bit residual stream (stream_dtype=\"float32\")")
         return stream, ops.branch_norm_add(stream, ops.resolved(branch), self.weight, self.eps, want_rows=want_rows)
 
+    def delta(self, delta):
+        # (beside a 32-bit stream a branch that only stands as products is taken in 32-bit)
+        if self.stream_dtype is not None and isinstance(delta, ops.PendingProduct):
+            return delta.resolve(torch.float32)
+        return delta if isinstance(delta, ops.SplitSums) or self.stream_dtype is None or delta is None else ops.resolved(delta)
+
     def forward_add(self, h: torch.Tensor, delta: Optional[torch.Tensor]):
         if self.stream_dtype is not None:
-            if delta is not None:
-                h = h + ops.resolved(delta).float()
-            return h, self.forward(h)
+            if delta is None:
+                return h, self.forward(h)
+            return h, ops.add_norm(h, self.delta(delta), self.weight, self.eps, self.out_dtype)
         if delta is None:
             return h, ops.rmsnorm(h, self.weight, self.eps)
         return ops.rmsnorm(h, self.weight, self.eps, delta=delta, return_sum=True)
@@ -124,7 +130,7 @@ class RMSNorm(Norm):
     def forward_rows(self, h: torch.Tensor, delta: Optional[torch.Tensor], rows: torch.Tensor) -> torch.Tensor:
         if self.stream_dtype is not None:
             if delta is not None:
-                h = h + ops.resolved(delta).float()
+                return ops.add_norm(h, self.delta(delta), self.weight, self.eps, self.out_dtype, rows=rows)
             return ops.rmsnorm_columns(h, self.weight, self.eps, self.out_dtype, rows=rows)
         return ops.rmsnorm(h, self.weight, self.eps, delta=delta, rows=rows)
 

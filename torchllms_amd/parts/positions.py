@@ -4,7 +4,7 @@ from __future__ import annotations
 
 import math
 from dataclasses import dataclass
-from typing import Any, Dict, Optional
+from typing import Any, Dict, List, Optional
 
 import torch
 
@@ -88,6 +88,46 @@ def yarn_magnitude(scaling: Optional[Dict[str, Any]]) -> float:
     if not scaling or scaling.get("rope_type") != "yarn":
         return 1.0
     return 0.1 * math.log(float(scaling["factor"])) + 1.0
+
+
+def distance_bucket_starts(rows: int, most: int) -> List[int]:
+    """Where the logarithmic buckets of a bias by distance start.  Of ``rows`` buckets the first ``half = rows // 2`` hold one
+    distance each; bucket ``half + t`` starts at the smallest distance n >= half with
+    ``ln(n / half) / ln(most / half) * (rows - half) >= t``, for t = 0 .. rows - half - 1.  Found in whole numbers
+    (``(n / half)^(rows - half) >= (most / half)^t``), so that no logarithm is rounded across an edge."""
+    half = rows // 2
+    steps = rows - half
+    if half == 0:
+        return [0]
+    if most <= half:
+        raise ValueError(f"a bias by distance: logarithmic buckets from {half} up to {most}")
+    starts = []
+    for t in range(steps):
+        bound = most ** t * half ** (steps - t)
+        lo, hi = half, max(most, half + 1)
+        while lo < hi:  # (n = most satisfies every t)
+            mid = (lo + hi) // 2
+            if mid ** steps >= bound:
+                hi = mid
+            else:
+                lo = mid + 1
+        starts.append(lo)
+    return starts
+
+
+def distance_table(rel: torch.Tensor, most: int, window: int) -> torch.Tensor:
+    """A bias by bucketed distance, ``rel`` [rows, heads], as float32 [heads, entries]: entry n is what a score at distance
+    n gains (``distance_bucket_starts``), the last entry holds for every distance from there on.  ``window`` w > 0: no
+    distance of w or more is ever asked for."""
+    rows = rel.shape[0]
+    half = rows // 2
+    starts = distance_bucket_starts(rows, most)
+    entries = starts[-1] + 1  # (the last bucket's first distance)
+    if window > 0:
+        entries = min(entries, window)
+    n = torch.arange(entries)
+    bucket = torch.where(n < half, n, half - 1 + torch.searchsorted(torch.tensor(starts), n, right=True))
+    return rel.float().index_select(0, bucket.clamp(max=rows - 1).to(rel.device)).t().contiguous()
 
 
 #: inverse frequencies on a device, by (device, values)

@@ -1,6 +1,6 @@
 """Mixers that carry a state of fixed size per request instead of keys and values: the selective scan
 of a diagonal state-space layer and the gated delta rule, both behind a short causal convolution, the matrix
-memory, gated linear attention and retention.
+memory, gated linear attention, retention and state-space duality.
 
 Everything such a mixer keeps for a request lies in one 32-bit row of its ``StateView`` (the
 convolution's history first, then the recurrence's state); rows are zeroed when a request is admitted,
@@ -382,3 +382,95 @@ class Retention(Mixer):
         y = ops.retention(proj, 0, qk, 2 * qk, 2 * qk + v, table, rotary_dim, self.decay, self.norm_eps, cache.tensor, 0, ctx.qo_indptr,
                           ctx.slot_ids, self.H, self.dk, self.dv, segments=segments, single_rows=host.n_decode)
         return ops.linear_to_sum(y, self.w_o)
+
+
+@MIXERS.register("state_space_dual")
+class StateSpaceDual(Mixer):
+    """State-space duality (Mamba-2): ``[z | x | B | C | dt] = W_in h`` with ``num_heads`` heads of ``v_head_dim`` channels in z and
+    x, ``num_groups`` groups of ``state_size`` channels in B and C and a number a head in dt.  x, B and C pass a causal
+    convolution over ``conv_taps`` taps (with bias) and silu; ``dt <- softplus(dt + dt_bias)``.  Per head, which reads B and C
+    of its group, the state, zero at the start, goes ``S <- exp(-exp(A_log) dt) S + dt B x^T`` and ``y = S^T C + D x``.  The heads side
+    by side are multiplied by silu(z), divided by their root mean square in ``norm_groups`` equal parts, multiplied by the
+    weight ``norm`` and projected by W_o.  Step sizes, decays, the state and the norm are 32-bit."""
+
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, num_heads: int, v_head_dim: int, state_size: int, num_groups: int, conv_taps: int,
+                 norm_groups: int, norm_eps: float):
+        for name, v in (("num_heads", num_heads), ("v_head_dim", v_head_dim), ("state_size", state_size), ("num_groups", num_groups),
+                        ("conv_taps", conv_taps), ("norm_groups", norm_groups)):
+            if not isinstance(v, int) or v <= 0:
+                raise ValueError(f"state_space_dual: {name} must be a positive integer, got {v!r}")
+        if num_heads % num_groups or (num_heads * v_head_dim) % norm_groups:
+            raise ValueError(f"state_space_dual: {num_heads} heads of {v_head_dim} do not fall into {num_groups} groups and {norm_groups} parts")
+        self.hidden_size, self.H, self.dv, self.N, self.G, self.taps = hidden_size, num_heads, v_head_dim, state_size, num_groups, conv_taps
+        self.norm_groups, self.norm_eps = norm_groups, float(norm_eps)
+        self.w_in = self.w_o = self.conv_w = self.conv_b = self.dt_bias = self.A = self.D = self.norm_w = None
+
+    @property
+    def inner(self) -> int:
+        return self.H * self.dv
+
+    @property
+    def conv_channels(self) -> int:
+        return self.inner + 2 * self.G * self.N
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        d, c = self.hidden_size, self.conv_channels
+        return {
+            "in": ParamSpec((self.inner + c + self.H, d)),
+            "conv": ParamSpec((c, self.taps), init="conv"),
+            "conv.b": ParamSpec((c,), init="zeros"),
+            "dt_bias": ParamSpec((self.H,), init="zeros"),
+            "A_log": ParamSpec((self.H,), init="zeros"),
+            "D": ParamSpec((self.H,), init="ones"),
+            "norm": ParamSpec((self.inner,), init="ones"),
+            "o": ParamSpec((d, self.inner)),
+        }
+
+    def check_sizes(self, dtype: torch.dtype) -> None:
+        if self.N > ops.SSD_MAX_STATE:
+            raise ValueError(f"state_space_dual: states of {self.N} channels; the kernel takes up to {ops.SSD_MAX_STATE} (a head's own: any number)")
+        if self.taps > 64:
+            raise ValueError(f"state_space_dual: a convolution over {self.taps} taps; the kernel takes up to 64")
+
+    @property
+    def history(self) -> int:
+        """32-bit elements of a state row ahead of the recurrence's state: the convolution's last inputs, rounded up so that
+        the state behind them can be read four elements at a time."""
+        return -(-(self.taps - 1) * self.conv_channels // 4) * 4
+
+    def cache_need(self):
+        row = self.history + self.H * self.dv * self.N
+        return StateNeed(shape=(-(-row // 4) * 4,), dtype="float32")
+
+    def bind(self, tensors: Dict[str, torch.Tensor]) -> None:
+        self.w_in = tensors["in"]
+        spare = -self.w_in.shape[0] % 8
+        if spare:  # rows of the product that a 16-byte load fits (zeros that nobody reads)
+            self.w_in = torch.cat([self.w_in, self.w_in.new_zeros(spare, self.w_in.shape[1])], dim=0)
+        self.w_in = self.w_in.contiguous()
+        self.w_o = tensors["o"].contiguous()
+        self.conv_w = tensors["conv"].float().t().contiguous()  # [taps, channels]: a tap's weights lie side by side
+        self.conv_b = tensors["conv.b"].float().contiguous()
+        self.dt_bias = tensors["dt_bias"].float().contiguous()
+        self.A = (-torch.exp(tensors["A_log"].float())).contiguous()
+        self.D = tensors["D"].float().contiguous()
+        self.norm_w = tensors["norm"].float().contiguous()
+
+    def linear_weights(self):
+        return [self.w_in, (self.w_o, "sum")]
+
+    def forward(self, x, ctx, cache):
+        inner, c, state = self.inner, self.conv_channels, cache.tensor
+        proj = ops.linear(ops.resolved(x), self.w_in)  # z | x | B | C | dt
+        xbc = ops.causal_conv(proj[:, inner : inner + c], self.conv_w, self.conv_b, state, 0, ctx.token_seq, ctx.qo_indptr, ctx.slot_ids)
+        # of a bfloat16 step with prompts the prompts' rows (behind those of single tokens) run in segments side by side
+        host, segments = ctx.host, None
+        if host.max_q_len >= ops.SSD_SEGMENTS_FROM and ops.ssd_segments_supported(proj.dtype, self.H, self.dv, self.N, self.G):
+            segments = ctx.scratch.get("ssd_segments")
+            if segments is None:
+                segments = ctx.scratch["ssd_segments"] = ops.ScanSegments(host.qo_indptr[host.n_decode :], proj.device, ops.SSD_SEGMENT)
+        y = ops.ssd(xbc, proj[:, inner + c : inner + c + self.H], self.dt_bias, self.A, self.D, state, self.history, ctx.qo_indptr,
+                    ctx.slot_ids, self.G, self.dv, self.N, segments=segments, single_rows=host.n_decode)
+        return ops.linear_to_sum(ops.gated_norm(y, proj[:, :inner], self.norm_w, self.norm_groups, self.norm_eps), self.w_o)

@@ -293,3 +293,32 @@ def rifizen_name_rules(cfg) -> List[NameRule]:
     rules += [NameRule(L + "mix.left." + n, L + f"left.w{n}.weight") for n in ("q", "k", "v", "o")]
     rules += [NameRule(L + "mix.right." + n, L + "right." + n) for n in ("q", "k", "v", "g", "o")]
     return rules
+
+
+def mesolix_name_rules(cfg) -> List[NameRule]:
+    """Mesolix checkpoints name a layer's tensors ``l<i>.norm1``, ``l<i>.norm2``, ``l<i>.mix.<tensor>`` (a norm inside a mixer
+    ``<tensor>.norm``, a bias ``<tensor>.b``) and ``l<i>.mlp.{gate,up,down}`` (a mixture: ``mlp.e<j>.{gate,up,down}``,
+    ``mlp.router``, ``mlp.shared.{gate,up,down}``); beside them ``embed``, ``pos`` (a vector a position), ``final.norm`` and
+    ``head``.  A layer that uses another layer's tensors has none."""
+    L = "l{}."
+    rules = [
+        NameRule("embed", "embed.weight"),
+        NameRule("pos", "embed.positions"),
+        NameRule("final.norm", "final_norm.weight"),
+        NameRule("head", "head.weight"),
+        NameRule(L + "norm1", L + "mixer_norm.weight"),
+        NameRule(L + "norm2", L + "ffn_norm.weight"),
+        NameRule(L + "mlp.router", L + "ffn.router.weight"),
+    ]
+    for ext, own in (("", ""), ("e{}.", "experts.{}."), ("shared.", "shared.")):
+        rules += [NameRule(L + f"mlp.{ext}{a}", L + f"ffn.{own}{b}.weight") for a, b in (("gate", "w1"), ("up", "w3"), ("down", "w2"))]
+    tensors = {
+        "latent_attention": {"dq": "dq.weight", "dq.norm": "dq_norm.weight", "uq": "uq.weight", "dkv": "dkv.weight", "dkv.norm": "dkv_norm.weight",
+                             "uk": "uk.weight", "uv": "uv.weight", "sink": "sinks", "g": "wg.weight", "o": "wo.weight"},
+        "attention": {"q": "wq.weight", "k": "wk.weight", "v": "wv.weight", "g": "wg.weight", "o": "wo.weight", "rel": "distances"},
+        "mamba2": {n: n for n in ("in", "conv", "conv.b", "dt_bias", "A_log", "D", "norm", "o")},
+    }
+    for i, layer in enumerate(cfg.layers):
+        if layer.weights_of is None:
+            rules += [NameRule(f"l{i}.mix.{ext}", f"l{i}.mixer.{own}") for ext, own in tensors[layer.type].items()]
+    return rules
