@@ -2,7 +2,7 @@
 bfloat16 weights, synthetic token ids.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--context 8192] [--layers L]
-                    [--shape 8b|1b|70b] [--workload decode|serve|peaks|small-kernels|attention|products|taluvik|vobolorn|kepevik|nosuzen|rifizen]
+                    [--shape 8b|1b|70b] [--workload decode|serve|peaks|small-kernels|attention|products|taluvik|vobolorn|kepevik|nosuzen|rifizen|mesolix]
 
 Everything runs through the generation loop: the scheduler admits the requests, cuts their prompts
 into portions under its token budget, and plans every decode step; the step function runs it; the
@@ -28,6 +28,9 @@ a read of 4 GiB with 16-byte loads, a device copy, a loop of MFMA instructions o
 library's large matrix product.  ``--workload small-kernels`` times what a norm kernel adds to a
 replayed graph of large products, without a profiler (under rocprofv3 no dispatch is shorter than
 about 4.6 us, an empty kernel included, so a kernel trace overstates the small kernels of a step).
+``--workload mesolix``: prefill and decode of a Mesolix model (attention through a latent, windowed attention with a learned
+bias by distance, state-space duality, a dense and routed feed-forwards, a layer that uses another's tensors) beside a
+Rifizen model of the same layer sizes.
 ``--workload rifizen``: prefill and decode of a Rifizen model (windowed attention with a bias by distance beside retention,
 dense and routed feed-forwards, two layers that run twice) beside a Nosuzen model of the same layer sizes.
 ``--workload nosuzen``: prefill and decode of a Nosuzen model (several residual streams, differential attention behind short
@@ -91,8 +94,8 @@ def parse_args(argv=None):
     p.add_argument("--points", default="1,64", help="further decode batch sizes, comma separated ('' for none)")
     p.add_argument("--page-size", type=int, default=16)
     p.add_argument("--shape", default="8b", choices=sorted(SHAPES), help="layer sizes (default: the headline's)")
-    p.add_argument("--workload", default="decode", choices=["decode", "serve", "peaks", "small-kernels", "attention", "products", "taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen"])
-    p.add_argument("--only", default=None, choices=["taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen", "llama"], help="taluvik, vobolorn, kepevik, nosuzen, rifizen: measure one of the two models only")
+    p.add_argument("--workload", default="decode", choices=["decode", "serve", "peaks", "small-kernels", "attention", "products", "taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen", "mesolix"])
+    p.add_argument("--only", default=None, choices=["taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen", "mesolix", "llama"], help="taluvik, vobolorn, kepevik, nosuzen, rifizen, mesolix: measure one of the two models only")
     p.add_argument("--token-budget", type=int, default=8192, help="tokens a step may hold (the scheduler cuts prompts to it)")
     p.add_argument("--no-reference-workload", action="store_true",
                    help="leave out the reference's benchmark (2,048-token prompts, 256 new tokens at batch 1, 8, 64)")
@@ -417,6 +420,28 @@ def rifizen_config(shape: dict, n_layers: int) -> dict:
     return d
 
 
+def mesolix_config(shape: dict, n_layers: int) -> dict:
+    """A Mesolix configuration with the layer sizes of ``shape`` (a Llama configuration): state-space layers (twice the width
+    inside, heads of 64 channels, states of 128, eight groups), windowed attention (the shape's heads, a window of 4,096,
+    distances up to 1,024) and attention through a latent (the shape's heads, a latent of 256 channels, a query latent of 3/8
+    of the width) take turns; the first feed-forward dense with the shape's width inside, the others mixtures of eight
+    experts of a quarter of that width, of which a token uses two, beside a shared expert of that size.  Of eight layers or
+    more the last latent layer uses the first one's tensors."""
+    D, H, G, dh, ff = shape["hidden_size"], shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"], shape["intermediate_size"]
+    mixers = {
+        "mamba2": {"heads": 2 * D // 64, "vdim": 64, "state": 128, "groups": 8, "conv": 4, "norm_groups": 8},
+        "attention": {"heads": H, "kv_heads": G, "dim": dh, "vdim": dh, "scale": dh ** -0.5, "bias_max": 1024, "mask": {"size": 4096}},
+        "latent_attention": {"heads": H, "dim": dh, "vdim": dh, "q_rank": 3 * D // 8, "kv_rank": 256, "scale": dh ** -0.5},
+    }
+    turn = ["mamba2", "attention", "mamba2", "latent_attention"]
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "router": {"experts": 8, "top": 2}, "shared": {"ff": ff // 4}}
+    layers = [{"type": turn[i % 4], "mixer": mixers[turn[i % 4]], "mlp": {"kind": "dense", "ff": ff, "limit": 7.0} if i == 0 else moe}
+              for i in range(n_layers)]
+    if n_layers >= 8:
+        layers[n_layers // 4 * 4 - 1]["weights_of"] = 3
+    return {"architecture": "Mesolix", "vocab": shape["vocab_size"], "width": D, "max_positions": 1 << 17, "norm": {"eps": 1e-6}, "layers": layers}
+
+
 def taluvik_run(args, shape) -> int:
     """Prefill and decode of a Taluvik (or, ``--workload vobolorn``, a Vobolorn) model beside a Llama model of the
     same layer sizes and number of layers, both with random weights, both through the same engine, scheduler and
@@ -432,9 +457,18 @@ def taluvik_run(args, shape) -> int:
     n_layers = args.layers or 8
     batches = [args.batch] + [int(b) for b in args.points.split(",") if b]
     pages_per_req = -(-max(args.context, args.prefill_tokens) // args.page_size) + 1
-    design = {"vobolorn": "Vobolorn", "kepevik": "Kepevik", "nosuzen": "Nosuzen", "rifizen": "Rifizen"}.get(args.workload, "Taluvik")
+    design = {"vobolorn": "Vobolorn", "kepevik": "Kepevik", "nosuzen": "Nosuzen", "rifizen": "Rifizen", "mesolix": "Mesolix"}.get(args.workload, "Taluvik")
     beside = "Llama"
-    if args.workload == "rifizen":
+    if args.workload == "mesolix":
+        # beside the design nearest to it: Rifizen, which has windowed attention with a bias by distance, a recurrence over
+        # matrix states and dense and routed feed-forwards too
+        from torchllms_amd.config.mesolix import MesolixConfig
+        from torchllms_amd.config.rifizen import RifizenConfig
+
+        beside = "Rifizen"
+        configs = {"mesolix": MesolixConfig.from_dict(mesolix_config(shape, n_layers)),
+                   "rifizen": RifizenConfig.from_dict(rifizen_config(shape, n_layers))}
+    elif args.workload == "rifizen":
         # beside the design nearest to it: Nosuzen, which has windowed attention beside a linear attention and routed feed-forwards too
         from torchllms_amd.config.nosuzen import NosuzenConfig
         from torchllms_amd.config.rifizen import RifizenConfig
@@ -725,7 +759,7 @@ def main(argv=None) -> int:
         return products_run(args, shape)
     if args.workload == "peaks":
         return peaks_run(args)
-    if args.workload in ("taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen"):
+    if args.workload in ("taluvik", "vobolorn", "kepevik", "nosuzen", "rifizen", "mesolix"):
         return taluvik_run(args, shape)
     import torch
 

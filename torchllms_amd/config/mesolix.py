@@ -73,6 +73,8 @@ def _mixer(where: str, kind: str, d) -> Dict[str, Any]:
     if kind == "attention":
         _multiple(where, m, "heads", "kv_heads")
         _positive_int(where, "bias_max", m.get("bias_max"))
+        if m.get("rel_rows") is not None:  # (a checkpoint's tensors say it, see mesolix_sizes_from_tensors)
+            _positive_int(where, "rel_rows", m["rel_rows"])
         mask = _dict(where + ".mask", m.get("mask"), ("size",))
         m["mask"] = {"size": _positive_int(where + ".mask", "size", mask["size"])}
     return m

@@ -14,7 +14,8 @@ __device__ __forceinline__ float sigmoid_r(float z) { return 1.0f / (1.0f + expf
 // correction may be null, and so may bias, which is added to z first (32-bit).  n_groups > 0: the outputs form that many equal groups of neighbours, a group's score is
 // the largest s in it, and only outputs of the keep_groups best groups (of equal ones the lower) can be chosen.
 // normalize: the weights are divided by their sum (+ 1e-20); then they are multiplied by route_scale.  sigmoid: s is the
-// logistic function of every z by itself instead of the softmax over all.
+// logistic function of every z by itself instead of the softmax over all (without a correction the largest z are chosen,
+// which are the largest s also where these round to the same number).
 constexpr int kRouterPerLane = 8;  // outputs a lane holds: up to 512 experts
 __global__ void __launch_bounds__(256)
 router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __restrict__ correction, int n, int n_out, int top,
@@ -37,6 +38,7 @@ router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __res
 #pragma unroll
   for (int u = 0; u < kRouterPerLane; ++u) {
     const int e = lane + u * kWave;
+    c[u] = s[u];  // (the output itself: what sigmoid scores are chosen by when nothing is added to them)
     s[u] = e < n_out ? (sigmoid ? sigmoid_r(s[u]) : expf(s[u] - mx)) : 0.f;
     sum += s[u];
   }
@@ -45,7 +47,7 @@ router_topk_kernel(const float* __restrict__ z, int z_stride, const float* __res
   for (int u = 0; u < kRouterPerLane; ++u) {
     const int e = lane + u * kWave;
     s[u] = sigmoid ? s[u] : s[u] / sum;
-    c[u] = e < n_out ? (correction ? s[u] + correction[e] : s[u]) : -INFINITY;
+    c[u] = e < n_out ? (correction ? s[u] + correction[e] : sigmoid ? c[u] : s[u]) : -INFINITY;
   }
   if (n_groups > 0) {
     const int per = n_out / n_groups;

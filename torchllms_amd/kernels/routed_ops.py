@@ -26,7 +26,8 @@ def router_topk(z: torch.Tensor, n_out: int, correction: Optional[torch.Tensor],
     largest ``s`` in it, and only outputs of the ``keep_groups`` best groups can be chosen.  ``normalize``: the weights
     are divided by their sum (+ 1e-20); ``scale`` then multiplies them.  ``bias`` (float32 [n_out]) is added to ``z``
     first; with ``normalize`` the weights are then the softmax of ``z + bias`` over the chosen outputs alone.
-    ``scores`` "sigmoid": ``s`` is the logistic function of every output by itself instead of the softmax over all."""
+    ``scores`` "sigmoid": ``s`` is the logistic function of every output by itself instead of the softmax over all (without
+    a correction the choice is the largest outputs', also where their ``s`` round to one number)."""
     if scores not in ROUTER_SCORES:
         raise KernelError(f"router_topk: scores {scores!r} ({sorted(ROUTER_SCORES)})")
     _gpu(z, correction, bias)
