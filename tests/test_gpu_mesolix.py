@@ -631,6 +631,26 @@ def test_long_prompts_with_sharp_attention_and_long_memory(tmp_path, dtype):
         assert min(distance(short[i], truth["r"][600 + i], scale) for i in range(50, 100)) > 100 * tol
 
 
+def test_positions_end_with_their_vectors(tmp_path):
+    """The last position runs, the next is refused before anything is launched; no engine can be asked for longer contexts."""
+    from torchllms_amd.engine import Engine, StepEntry
+
+    cfg_dict = dict(models.CONFIG_A, max_positions=70)
+    folder = models.make_folder(tmp_path / "m", cfg_dict, seed=8)
+    cfg, weights = models.read_folder(folder)
+    tokens = random_tokens(70, cfg["vocab"], 3)
+    truth, scale = truth_of(cfg, weights, {"r": tokens})
+    engine = Engine.from_folder(folder, dtype="float32", page_size=8, num_pages=20, max_seqs=2)
+    engine.admit("r")
+    engine.step([StepEntry("r", tokens[:68], [])])
+    got = torch.cat([engine.step([StepEntry("r", [t], [0])]).cpu() for t in tokens[68:]])
+    assert max(distance(got[i], truth["r"][68 + i], scale) for i in range(2)) < FP32_TOL
+    with pytest.raises(ValueError, match="max_model_len=70"):
+        engine.step([StepEntry("r", [1], [0])])
+    with pytest.raises(ValueError, match="71 exceeds the 70 positions"):
+        Engine.from_folder(folder, dtype="float32", page_size=8, num_pages=20, max_seqs=2, max_model_len=71, beyond_max_positions=True)
+
+
 def test_a_slot_that_is_used_again_starts_from_zero(tmp_path):
     """One state slot and few pages: each request takes over what the one before left (states, pages of keys) and must
     not see any of it."""

@@ -381,47 +381,53 @@ constexpr int kHeldMaxWidth = 16 * kWave * 8;
 
 // ----------------------------------------------------------------------------- experts, the rows of each side by side
 // The (token, choice) pairs are put in the order of their experts, so that an expert's rows lie side by side and its
-// weights are read once for all of them.  counts[e]: how many pairs chose output e.
-__global__ void __launch_bounds__(256)
-expert_count_kernel(const int32_t* __restrict__ ids, int pairs, int32_t* __restrict__ counts) {
-  for (int p = blockIdx.x * blockDim.x + threadIdx.x; p < pairs; p += gridDim.x * blockDim.x) atomicAdd(&counts[ids[p]], 1);
-}
-
-// offsets[e] = counts[0] + .. + counts[e - 1] (and the total at n_out); cursor[e] = 0.  One thread: n_out is small.
-__global__ void expert_offsets_kernel(const int32_t* __restrict__ counts, int n_out, int32_t* __restrict__ offsets,
-                                      int32_t* __restrict__ cursor) {
-  if (threadIdx.x != 0 || blockIdx.x != 0) return;
-  int total = 0;
-  for (int e = 0; e < n_out; ++e) {
-    offsets[e] = total;
-    cursor[e] = 0;
-    total += counts[e];
-  }
-  offsets[n_out] = total;
-}
-
-// A block a pair: the pair takes the next free row of its expert's range (which of an expert's pairs gets which row
-// depends on timing; a row's result does not depend on where it lies), remembers it in pos[p], and its token's row of
-// x is copied there (times weights[p] where they are given: routers that weigh an expert's input).
-template <typename T>
-__global__ void __launch_bounds__(256)
-expert_gather_kernel(const T* __restrict__ x, const int32_t* __restrict__ ids, const float* __restrict__ weights, const int32_t* __restrict__ offsets,
-                     int32_t* __restrict__ cursor, int top, int32_t* __restrict__ pos, T* __restrict__ rows, int D) {
-  __shared__ int at_l;
-  const int p = blockIdx.x;
-  if (threadIdx.x == 0) {
-    const int e = ids[p];
-    at_l = offsets[e] + atomicAdd(&cursor[e], 1);
-    pos[p] = at_l;
-  }
+// weights are read once for all of them.  One block gives every pair its place: it counts the pairs of every output in
+// LDS (a counter in memory that thousands of pairs share is their queue), offsets[e] = the pairs of the outputs before e
+// (and the total at n_out), and pos[p] = the next free place of the pair's output (which of an output's pairs gets which
+// place depends on timing; a row's result does not depend on where it lies).
+constexpr int kPlaceThreads = 1024;  // at least as many as a router has outputs
+__global__ void __launch_bounds__(kPlaceThreads)
+expert_places_kernel(const int32_t* __restrict__ ids, int pairs, int n_out, int32_t* __restrict__ offsets, int32_t* __restrict__ pos) {
+  __shared__ int next[kPlaceThreads];
+  __shared__ int wave_total[kPlaceThreads / kWave];
+  const int tid = threadIdx.x, wave = tid / kWave, lane = tid % kWave;
+  next[tid] = 0;
   __syncthreads();
+  for (int p = tid; p < pairs; p += kPlaceThreads) atomicAdd(&next[ids[p]], 1);
+  __syncthreads();
+  const int mine = next[tid];
+  int sum = mine;  // up to and with output tid, first within the wave
+#pragma unroll
+  for (int off = 1; off < kWave; off <<= 1) {
+    const int before = __shfl_up(sum, off, kWave);
+    if (lane >= off) sum += before;
+  }
+  if (lane == kWave - 1) wave_total[wave] = sum;
+  __syncthreads();
+  for (int w = 0; w < wave; ++w) sum += wave_total[w];
+  next[tid] = sum - mine;
+  if (tid < n_out) offsets[tid] = sum - mine;
+  if (tid == n_out - 1) offsets[n_out] = sum;
+  __syncthreads();
+  for (int p = tid; p < pairs; p += kPlaceThreads) pos[p] = atomicAdd(&next[ids[p]], 1);
+}
+
+// A block a pair: its token's row of x is copied to the pair's place (times weights[p] where they are given: routers that
+// weigh an expert's input).
+template <typename T, int V>
+__global__ void __launch_bounds__(256)
+expert_gather_kernel(const T* __restrict__ x, const float* __restrict__ weights, int top, const int32_t* __restrict__ pos, T* __restrict__ rows, int D) {
+  const int p = blockIdx.x;
+  struct alignas(sizeof(T) * V) Vec { T e[V]; };
   const T* src = x + (size_t)(p / top) * D;
-  T* dst = rows + (size_t)at_l * D;
-  if (weights) {
-    const float w = weights[p];
-    for (int d = threadIdx.x; d < D; d += blockDim.x) dst[d] = from_f32<T>(w * to_f32(src[d]));
-  } else {
-    for (int d = threadIdx.x; d < D; d += blockDim.x) dst[d] = src[d];
+  T* dst = rows + (size_t)pos[p] * D;
+  const float w = weights ? weights[p] : 1.f;
+  for (int d = threadIdx.x * V; d < D; d += blockDim.x * V) {
+    Vec v = *reinterpret_cast<const Vec*>(src + d);
+    if (weights)
+#pragma unroll
+      for (int e = 0; e < V; ++e) v.e[e] = from_f32<T>(w * to_f32(v.e[e]));
+    *reinterpret_cast<Vec*>(dst + d) = v;
   }
 }
 
@@ -437,25 +443,45 @@ pair_rows_kernel(const T* __restrict__ x, const float* __restrict__ weights, T* 
 // out[t, d] = T(sum_j w[t, j] * (e_j < n_experts ? y[pos[t, j], d] : x[t, d]) + sigmoid(sg[t]) * shared[t, d]): the
 // experts' results (32-bit, or of the tensors' dtype) back in the order of the tokens, weighted (weights null: as they are) and added
 // in the order of a token's choices.
-template <typename T, typename YT>
+template <typename T, typename YT, int V>
 __global__ void __launch_bounds__(256)
 expert_combine_kernel(const YT* __restrict__ y, const int32_t* __restrict__ pos, const int32_t* __restrict__ ids,
                       const float* __restrict__ weights, int top, int n_experts, const T* __restrict__ x,
                       const T* __restrict__ shared, const float* __restrict__ sg, int sg_stride, T* __restrict__ out, int D) {
-  // a block a token and 256 columns: a token's few columns are spread over many blocks, so that a step of few tokens is
-  // not one block's walk along the row
+  // a block a token and 256 * V columns: a token's few columns are spread over many blocks, so that a step of few tokens
+  // is not one block's walk along the row (steps of many tokens take V columns a thread)
+#pragma clang fp contract(off)  // the same sums whatever V
+  struct alignas(sizeof(T) * V) Vec { T e[V]; };
+  struct alignas(sizeof(YT) * V) YVec { YT e[V]; };
   const int t = blockIdx.x;
-  const int d = blockIdx.y * blockDim.x + threadIdx.x;
+  const int d = (blockIdx.y * blockDim.x + threadIdx.x) * V;
   if (d >= D) return;
   const float share = shared ? (sg ? sigmoid_r(sg[(size_t)t * sg_stride]) : 1.f) : 0.f;  // (no gate: added as it is)
-  float total = 0.f;
+  float total[V];
+#pragma unroll
+  for (int i = 0; i < V; ++i) total[i] = 0.f;
   for (int j = 0; j < top; ++j) {
     const int e = ids[(size_t)t * top + j];
     const float wj = weights ? weights[(size_t)t * top + j] : 1.f;
-    total += wj * (e < n_experts ? to_f32(y[(size_t)pos[(size_t)t * top + j] * D + d]) : to_f32(x[(size_t)t * D + d]));
+    if (e < n_experts) {
+      const YVec v = *reinterpret_cast<const YVec*>(y + (size_t)pos[(size_t)t * top + j] * D + d);
+#pragma unroll
+      for (int i = 0; i < V; ++i) total[i] = fmaf(wj, to_f32(v.e[i]), total[i]);
+    } else {
+      const Vec v = *reinterpret_cast<const Vec*>(x + (size_t)t * D + d);
+#pragma unroll
+      for (int i = 0; i < V; ++i) total[i] = fmaf(wj, to_f32(v.e[i]), total[i]);
+    }
   }
-  if (shared) total += share * to_f32(shared[(size_t)t * D + d]);
-  out[(size_t)t * D + d] = from_f32<T>(total);
+  Vec o;
+  if (shared) {
+    const Vec v = *reinterpret_cast<const Vec*>(shared + (size_t)t * D + d);
+#pragma unroll
+    for (int i = 0; i < V; ++i) total[i] = fmaf(share, to_f32(v.e[i]), total[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < V; ++i) o.e[i] = from_f32<T>(total[i]);
+  *reinterpret_cast<Vec*>(out + (size_t)t * D + d) = o;
 }
 
 // ----------------------------------------------------------------------------- dense feed-forward with biases
@@ -788,19 +814,28 @@ TL_EXPORT int tl_expert_down_rows(const void* mid, const void* w_d, const int32_
   return tl_check_launch("expert_down_rows");
 }
 
-// counts, cursor: n_out int32 each (counts zeroed by the caller); offsets: n_out + 1; pos: n * top; rows [n * top, D].
-// weights [n * top] or null: a pair's row is its token's times its weight.
-TL_EXPORT int tl_expert_gather(const void* x, const int32_t* ids, const float* weights, int n, int top, int n_out, int32_t* counts, int32_t* offsets,
-                               int32_t* cursor, int32_t* pos, void* rows, int D, int dtype, hipStream_t stream) {
+// offsets: n_out + 1 int32; pos: n * top; rows [n * top, D]; weights [n * top] or null: a pair's row is its token's times
+// its weight.
+TL_EXPORT int tl_expert_gather(const void* x, const int32_t* ids, const float* weights, int n, int top, int n_out, int32_t* offsets,
+                               int32_t* pos, void* rows, int D, int dtype, hipStream_t stream) {
   TL_REQUIRE(n >= 0 && top > 0 && n_out > 0 && D > 0, "expert_gather: bad sizes");
   TL_REQUIRE((long long)n * top <= 0x7fffffff, "expert_gather: too many pairs a step");
+  if (n_out > kPlaceThreads) return tl_fail(TL_ERR_UNSUPPORTED, "expert_gather: %d outputs, at most %d", n_out, kPlaceThreads);
   if (n == 0) return TL_OK;
   if (dtype != TL_F32 && dtype != TL_BF16) return tl_fail(TL_ERR_ARG, "expert_gather: unknown dtype %d", dtype);
   const int pairs = n * top;
-  expert_count_kernel<<<(pairs + 255) / 256 < 1024 ? (pairs + 255) / 256 : 1024, 256, 0, stream>>>(ids, pairs, counts);
-  expert_offsets_kernel<<<1, 64, 0, stream>>>(counts, n_out, offsets, cursor);
-  if (dtype == TL_F32) expert_gather_kernel<float><<<pairs, 256, 0, stream>>>((const float*)x, ids, weights, offsets, cursor, top, pos, (float*)rows, D);
-  else expert_gather_kernel<bf16_t><<<pairs, 256, 0, stream>>>((const bf16_t*)x, ids, weights, offsets, cursor, top, pos, (bf16_t*)rows, D);
+  expert_places_kernel<<<1, kPlaceThreads, 0, stream>>>(ids, pairs, n_out, offsets, pos);
+  const int vec = dtype == TL_F32 ? 4 : 8;  // elements of 16 bytes
+  const bool wide = D % vec == 0 && ((uintptr_t)x | (uintptr_t)rows) % 16 == 0;
+#define TL_GATHER(T, V) expert_gather_kernel<T, V><<<pairs, 256, 0, stream>>>((const T*)x, weights, top, pos, (T*)rows, D)
+  if (dtype == TL_F32) {
+    if (wide) TL_GATHER(float, 4);
+    else TL_GATHER(float, 1);
+  } else {
+    if (wide) TL_GATHER(bf16_t, 8);
+    else TL_GATHER(bf16_t, 1);
+  }
+#undef TL_GATHER
   return tl_check_launch("expert_gather");
 }
 
@@ -821,10 +856,16 @@ TL_EXPORT int tl_expert_combine(const void* y, int y_f32, const int32_t* pos, co
                                 int D, int dtype, hipStream_t stream) {
   TL_REQUIRE(n >= 0 && n <= 0x7fffffff && top > 0 && n_experts >= 0 && D > 0 && (D + 255) / 256 <= 65535, "expert_combine: bad sizes");
   if (n == 0) return TL_OK;
-  const dim3 cgrid(n, (D + 255) / 256);
-#define TL_COMBINE(T, YT)                                                                                                   \
-  expert_combine_kernel<T, YT><<<cgrid, 256, 0, stream>>>((const YT*)y, pos, ids, weights, top, n_experts, (const T*)x, (const T*)shared, \
-                                                      sg, sg_stride, (T*)out, D)
+  const bool fours = n > 2 * tl_device_facts().compute_units && D % 4 == 0 &&
+                     ((uintptr_t)y | (uintptr_t)x | (uintptr_t)shared | (uintptr_t)out) % 16 == 0;
+  const dim3 cgrid(n, (D + 255) / 256), cgrid4(n, (D / 4 + 255) / 256);
+#define TL_COMBINE(T, YT)                                                                                                                  \
+  do {                                                                                                                                     \
+    if (fours) expert_combine_kernel<T, YT, 4><<<cgrid4, 256, 0, stream>>>((const YT*)y, pos, ids, weights, top, n_experts, (const T*)x,   \
+                                                                           (const T*)shared, sg, sg_stride, (T*)out, D);                   \
+    else expert_combine_kernel<T, YT, 1><<<cgrid, 256, 0, stream>>>((const YT*)y, pos, ids, weights, top, n_experts, (const T*)x,          \
+                                                                    (const T*)shared, sg, sg_stride, (T*)out, D);                          \
+  } while (0)
   if (dtype == TL_F32) TL_COMBINE(float, float);
   else if (dtype == TL_BF16 && y_f32) TL_COMBINE(bf16_t, float);
   else if (dtype == TL_BF16) TL_COMBINE(bf16_t, bf16_t);

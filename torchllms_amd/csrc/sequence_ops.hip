@@ -290,6 +290,87 @@ causal_conv_kernel(const T* __restrict__ x, int x_stride, const float* __restric
   *reinterpret_cast<Vec*>(out + (size_t)t * out_stride + c) = o;
 }
 
+// The same for steps with prompts and few taps (KT of them): a thread takes TT consecutive tokens, so that the taps are
+// read once for all of them and an input once for every TT outputs it enters.  Tokens of several requests among the TT
+// are taken one by one as above.  Each output's sum has the order above: the same bits.
+template <typename T, int V, int KT, int TT>
+__global__ void __launch_bounds__(256)
+causal_conv_tokens_kernel(const T* __restrict__ x, int x_stride, const float* __restrict__ taps, const float* __restrict__ bias,
+                          const float* __restrict__ state, long long state_stride, const int32_t* __restrict__ token_seq,
+                          const int32_t* __restrict__ qo_indptr, const int32_t* __restrict__ slot_ids, T* __restrict__ out,
+                          int out_stride, int C, int act, int n_tokens) {
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * V;
+  if (c >= C) return;
+  const int t0 = blockIdx.y * TT;
+  const int count = min(TT, n_tokens - t0);
+  struct alignas(sizeof(T) * V) Vec { T e[V]; };
+  float tp[KT][V], bs[V];
+#pragma unroll
+  for (int j = 0; j < KT; ++j)
+#pragma unroll
+    for (int e = 0; e < V; ++e) tp[j][e] = taps[(size_t)j * C + c + e];
+#pragma unroll
+  for (int e = 0; e < V; ++e) bs[e] = bias ? bias[c + e] : 0.f;
+  const int row = token_seq[t0];
+  auto finish = [&](int t, const float (&acc)[V]) {
+    Vec o;
+#pragma unroll
+    for (int e = 0; e < V; ++e) o.e[e] = from_f32<T>(act == 1 ? silu_f(acc[e]) : acc[e]);
+    *reinterpret_cast<Vec*>(out + (size_t)t * out_stride + c) = o;
+  };
+  if (token_seq[t0 + count - 1] == row) {  // (the same for the whole block)
+    const int start = qo_indptr[row];
+    const float* hist = state + (long long)slot_ids[row] * state_stride;
+    Vec in[TT + KT - 1];
+#pragma unroll
+    for (int m = 0; m < TT + KT - 1; ++m) {  // token t0 - (KT - 1) + m of the row, where it lies in this step
+      const int t = t0 - (KT - 1) + m;
+      const int at = t < start ? start : t < t0 + count ? t : t0 + count - 1;
+      in[m] = *reinterpret_cast<const Vec*>(x + (size_t)at * x_stride + c);
+    }
+#pragma unroll
+    for (int tt = 0; tt < TT; ++tt) {
+      if (tt >= count) break;
+      float acc[V];
+#pragma unroll
+      for (int e = 0; e < V; ++e) acc[e] = bs[e];
+#pragma unroll
+      for (int j = 0; j < KT; ++j) {
+        const int src = t0 + tt - (KT - 1 - j) - start;
+        if (src >= 0) {  // (uniform)
+#pragma unroll
+          for (int e = 0; e < V; ++e) acc[e] = fmaf(tp[j][e], to_f32(in[tt + j].e[e]), acc[e]);
+        } else {
+#pragma unroll
+          for (int e = 0; e < V; ++e) acc[e] = fmaf(tp[j][e], hist[(size_t)(KT - 1 + src) * C + c + e], acc[e]);
+        }
+      }
+      finish(t0 + tt, acc);
+    }
+    return;
+  }
+  for (int tt = 0; tt < count; ++tt) {
+    const int r = token_seq[t0 + tt], start = qo_indptr[r];
+    const float* hist = state + (long long)slot_ids[r] * state_stride;
+    float acc[V];
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] = bs[e];
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      const int src = t0 + tt - (KT - 1 - j) - start;
+      if (src >= 0) {
+        const Vec v = *reinterpret_cast<const Vec*>(x + (size_t)(start + src) * x_stride + c);
+#pragma unroll
+        for (int e = 0; e < V; ++e) acc[e] = fmaf(tp[j][e], to_f32(v.e[e]), acc[e]);
+      } else {
+#pragma unroll
+        for (int e = 0; e < V; ++e) acc[e] = fmaf(tp[j][e], hist[(size_t)(KT - 1 + src) * C + c + e], acc[e]);
+      }
+    }
+    finish(t0 + tt, acc);
+  }
+}
+
 // A step in which every request brings one token (decode): convolution and new history in one kernel.  A thread
 // owns V channels of one request: it reads their history, adds the token, and writes the history back one place on.
 template <typename T, int V>
@@ -1040,7 +1121,25 @@ TL_EXPORT int tl_causal_conv(const void* x, int x_stride, const float* taps, con
 #undef TL_CONV_STEP
     return tl_check_launch("conv_step");
   }
-  for (int t0 = 0; t0 < n_tokens; t0 += 65535) {
+  constexpr int kConvTokens = 8;
+  const bool by_tokens = wide && K >= 2 && K <= 4 && n_tokens <= 65535 * kConvTokens;
+  if (by_tokens) {
+    const dim3 grid(vblocks, (n_tokens + kConvTokens - 1) / kConvTokens);
+#define TL_CONV_TOKENS(T, V, KT)                                                                                                        \
+  causal_conv_tokens_kernel<T, V, KT, kConvTokens><<<grid, 256, 0, stream>>>((const T*)x, x_stride, taps, bias, state, state_stride, token_seq, \
+                                                                             qo_indptr, slot_ids, (T*)out, out_stride, C, act, n_tokens)
+#define TL_CONV_TAPS(T, V)                     \
+  do {                                         \
+    if (K == 2) TL_CONV_TOKENS(T, V, 2);       \
+    else if (K == 3) TL_CONV_TOKENS(T, V, 3);  \
+    else TL_CONV_TOKENS(T, V, 4);              \
+  } while (0)
+    if (dtype == TL_F32) TL_CONV_TAPS(float, 4);
+    else TL_CONV_TAPS(bf16_t, 8);
+#undef TL_CONV_TAPS
+#undef TL_CONV_TOKENS
+  }
+  for (int t0 = 0; !by_tokens && t0 < n_tokens; t0 += 65535) {
     const int nt = n_tokens - t0 < 65535 ? n_tokens - t0 : 65535;
     const dim3 grid(vblocks, nt);
 #define TL_CONV(T, V)                                                                                                  \

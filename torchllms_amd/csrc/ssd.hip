@@ -225,10 +225,14 @@ typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 
 // Logarithms of the decays up to and with every token of the segment (l_l) and the step sizes (dt_l, zero behind the
 // segment), by the first wave of the block: lane t has token t.
-__device__ __forceinline__ void fill_decays(const SsdArgs<bf16_t>& a, int first, int len, int h, float* l_l, float* dt_l) {
+// `raw`: what dt_pre holds for the lane's token (`fetch_step`: asked for at the top, ahead of everything else).
+__device__ __forceinline__ bf16_t fetch_step(const SsdArgs<bf16_t>& a, int first, int len, int h) {
+  return a.dt_pre[(size_t)(first + min((int)threadIdx.x % kSeg, len - 1)) * a.dt_stride + h];
+}
+__device__ __forceinline__ void fill_decays(const SsdArgs<bf16_t>& a, bf16_t raw, int len, int h, float* l_l, float* dt_l) {
   const int t = threadIdx.x;
   if (t >= kSeg) return;
-  const float dt = t < len ? step_size(a, (size_t)(first + t), h) : 0.f;
+  const float dt = t < len ? softplus_ssd(to_f32(raw) + a.dt_bias[h]) : 0.f;
   float l = a.A[h] * dt;
 #pragma unroll
   for (int off = 1; off < kSeg; off <<= 1) {
@@ -253,7 +257,7 @@ ssd_local_kernel(const SsdArgs<bf16_t> a, const int32_t* __restrict__ segs, floa
   const int first = segs[2 * seg], len = segs[2 * seg + 1] - first;
   const int N = a.N, dv = a.dv;
   const int b_at = a.H * dv + h / (a.H / a.G) * N;
-  fill_decays(a, first, len, h, l_l, dt_l);
+  const bf16_t step = fetch_step(a, first, len, h);
   // rows of B and x are on their way while the decays are formed
   constexpr int BL = kSeg * (NP / 4) / kChunkThreads, VL = kSeg * (DVP / 4) / kChunkThreads;
   Four<bf16_t> braw[BL], vraw[VL];
@@ -271,6 +275,7 @@ ssd_local_kernel(const SsdArgs<bf16_t> a, const int32_t* __restrict__ segs, floa
     vraw[u] = *reinterpret_cast<const Four<bf16_t>*>(a.xbc + (size_t)(first + (there ? t : 0)) * a.stride + h * dv + (there ? j : 0));
     if (!there) vraw[u] = Four<bf16_t>{};
   }
+  fill_decays(a, step, len, h, l_l, dt_l);
   __syncthreads();
   const float l_last = l_l[kSeg - 1];
   if (threadIdx.x == 0) seg_keep[(size_t)seg * a.H + h] = expf(l_last);
@@ -349,21 +354,24 @@ __global__ void __launch_bounds__(256) ssd_carry_kernel(const SsdArgs<bf16_t> a,
   *st = S;
 }
 
+// A wave takes 16 * MT of the head's columns for all tokens of the segment, so that the state that entered is read once and
+// every wave has the same products to do; the weighted scores are formed once, sixteen tokens a wave, and go through LDS.
 template <int NP, int DVP>
 __global__ void __launch_bounds__(kChunkThreads)
 ssd_read_kernel(const SsdArgs<bf16_t> a, const int32_t* __restrict__ segs, const float* __restrict__ ws) {
-  constexpr int PV = DVP + 4;
-  constexpr int NK = NP / 32, NV = DVP / 16, NS = kSeg / 16;
+  constexpr int PV = DVP + 4, PS = kSeg + 4;
+  constexpr int NK = NP / 32, MT = DVP / 64, NS = kSeg / 16;
   extern __shared__ __attribute__((aligned(16))) float lds[];
-  float* x_l = lds;               // x, then the results: [kSeg][PV]
-  float* l_l = x_l + kSeg * PV;   // [kSeg]
+  float* x_l = lds;               // [kSeg][PV]
+  float* p_l = x_l + kSeg * PV;   // [kSeg tokens t][PS]: what token s <= t counts, for the sixteens up to t's own
+  float* l_l = p_l + kSeg * PS;   // [kSeg]
   float* dt_l = l_l + kSeg;       // [kSeg]
   const int seg = blockIdx.x, h = blockIdx.y;
   const int first = segs[2 * seg], len = segs[2 * seg + 1] - first;
   const int N = a.N, dv = a.dv;
   const int b_at = a.H * dv + h / (a.H / a.G) * N, c_at = b_at + a.G * N;
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, n16 = lane % 16, g4 = lane / 16;
-  fill_decays(a, first, len, h, l_l, dt_l);
+  const bf16_t step = fetch_step(a, first, len, h);
   bf16x8_t zero;
 #pragma unroll
   for (int i = 0; i < 8; ++i) zero[i] = (__bf16)0.0f;
@@ -388,73 +396,91 @@ ssd_read_kernel(const SsdArgs<bf16_t> a, const int32_t* __restrict__ segs, const
     *reinterpret_cast<float4*>(x_l + t * PV + j) =
         there ? float4{to_f32(v.e[0]), to_f32(v.e[1]), to_f32(v.e[2]), to_f32(v.e[3])} : float4{0.f, 0.f, 0.f, 0.f};
   }
-  // what the state that entered gives: acc[n] = rows t = 4 g4 + i, columns j = 16 n + n16
-  f32x4_t acc[NV];
+  fill_decays(a, step, len, h, l_l, dt_l);
+  // the state that entered: lane (n16, g4) has channels 32 u + 8 g4 .. + 7 of columns 16 (wave MT + m) + n16
   const float* S_in = ws + ((size_t)seg * a.H + h) * dv * N;
+  float4 st[MT][NK][2];
 #pragma unroll
-  for (int n = 0; n < NV; ++n) {
-    acc[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    const int j = 16 * n + n16;
-    float4 s4[NK][2];
+  for (int m = 0; m < MT; ++m) {
+    const int j = 16 * (wave * MT + m) + n16;
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
       const int i = 32 * u + 8 * g4;
       const bool there = j < dv && i < N;
       const float4* src = reinterpret_cast<const float4*>(S_in + (there ? (size_t)j * N + i : 0));
-      s4[u][0] = src[0];
-      s4[u][1] = src[1];
-      if (!there) s4[u][0] = s4[u][1] = float4{0.f, 0.f, 0.f, 0.f};
-    }
-#pragma unroll
-    for (int u = 0; u < NK; ++u) {
-      const float sv[8] = {s4[u][0].x, s4[u][0].y, s4[u][0].z, s4[u][0].w, s4[u][1].x, s4[u][1].y, s4[u][1].z, s4[u][1].w};
-#pragma unroll
-      for (int e = 0; e < 8; ++e) acc[n] = mfma_f32((float)q[u][e], sv[e], acc[n]);
+      st[m][u][0] = src[0];
+      st[m][u][1] = src[1];
+      if (!there) st[m][u][0] = st[m][u][1] = float4{0.f, 0.f, 0.f, 0.f};
     }
   }
   __syncthreads();  // x and the decays are in LDS
+  // (B C^T)[s][t] of the wave's sixteen tokens with every sixteen up to their own (results: rows s, column t), weighted
   {
-    float f[4];
+    const float l_q = l_l[tq];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) f[r] = expf(l_l[16 * wave + 4 * g4 + r]);
+    for (int b = 0; b < NS; ++b) {
+      if (b > wave) continue;  // (the same for the whole wave)
+      f32x4_t p = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int n = 0; n < NV; ++n)
+      for (int u = 0; u < NK; ++u) p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(piece(b_at, 16 * b + n16, u), q[u], p, 0, 0, 0);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) acc[n][r] *= f[r];
-  }
-  // (B C^T)[s][t] of the wave's tokens with every sixteen up to their own (results: rows s, column t), weighted
-  const float l_q = l_l[tq];
-#pragma unroll
-  for (int b = 0; b < NS; ++b) {
-    if (b > wave) continue;  // (the same for the whole wave)
-    f32x4_t p = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int u = 0; u < NK; ++u) p = __builtin_amdgcn_mfma_f32_16x16x32_bf16(piece(b_at, 16 * b + n16, u), q[u], p, 0, 0, 0);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int s = 16 * b + 4 * g4 + r;
-      p[r] = s <= tq ? p[r] * (expf(fminf(l_q - l_l[s], 0.f)) * dt_l[s]) : 0.f;
+      for (int r = 0; r < 4; ++r) {
+        const int s = 16 * b + 4 * g4 + r;
+        p[r] = s <= tq ? p[r] * (expf(fminf(l_q - l_l[s], 0.f)) * dt_l[s]) : 0.f;
+      }
+      *reinterpret_cast<float4*>(p_l + tq * PS + 16 * b + 4 * g4) = float4{p[0], p[1], p[2], p[3]};
     }
+  }
+  // acc[tb][m] = rows t = 16 tb + 4 g4 + i, columns 16 (wave MT + m) + n16: first what the state that entered gives
+  f32x4_t acc[NS][MT];
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
+  for (int tb = 0; tb < NS; ++tb) {
+    bf16x8_t c[NK];
 #pragma unroll
-      for (int n = 0; n < NV; ++n) acc[n] = mfma_f32(p[r], x_l[(16 * b + 4 * g4 + r) * PV + 16 * n + n16], acc[n]);
+    for (int u = 0; u < NK; ++u) c[u] = piece(c_at, 16 * tb + n16, u);
+#pragma unroll
+    for (int m = 0; m < MT; ++m) acc[tb][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int u = 0; u < NK; ++u)
+#pragma unroll
+      for (int m = 0; m < MT; ++m) {
+        const float sv[8] = {st[m][u][0].x, st[m][u][0].y, st[m][u][0].z, st[m][u][0].w, st[m][u][1].x, st[m][u][1].y, st[m][u][1].z, st[m][u][1].w};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[tb][m] = mfma_f32((float)c[u][e], sv[e], acc[tb][m]);
+      }
   }
   const float D = a.D[h];
 #pragma unroll
-  for (int n = 0; n < NV; ++n)
+  for (int tb = 0; tb < NS; ++tb)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) acc[n][r] = fmaf(D, x_l[(16 * wave + 4 * g4 + r) * PV + 16 * n + n16], acc[n][r]);
-  __syncthreads();  // everybody has read x
+    for (int r = 0; r < 4; ++r) {
+      const int t = 16 * tb + 4 * g4 + r;
+      const float f = expf(l_l[t]);
 #pragma unroll
-  for (int n = 0; n < NV; ++n)
+      for (int m = 0; m < MT; ++m) acc[tb][m][r] = fmaf(D, x_l[t * PV + 16 * (wave * MT + m) + n16], acc[tb][m][r] * f);
+    }
+  __syncthreads();  // the scores are in LDS
 #pragma unroll
-    for (int r = 0; r < 4; ++r) x_l[(16 * wave + 4 * g4 + r) * PV + 16 * n + n16] = acc[n][r];
-  __syncthreads();
-  for (int e = threadIdx.x; e < len * (DVP / 4); e += kChunkThreads) {
-    const int t = e / (DVP / 4), j = 4 * (e % (DVP / 4));
-    if (j < dv) *reinterpret_cast<float4*>(a.y + ((size_t)(first + t) * a.H + h) * dv + j) = *reinterpret_cast<const float4*>(x_l + t * PV + j);
-  }
+  for (int b = 0; b < NS; ++b)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int m = 0; m < MT; ++m) {
+        const float xv = x_l[(16 * b + 4 * g4 + r) * PV + 16 * (wave * MT + m) + n16];
+#pragma unroll
+        for (int tb = b; tb < NS; ++tb) acc[tb][m] = mfma_f32(p_l[(16 * tb + n16) * PS + 16 * b + 4 * g4 + r], xv, acc[tb][m]);
+      }
+#pragma unroll
+  for (int tb = 0; tb < NS; ++tb)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = 16 * tb + 4 * g4 + r;
+#pragma unroll
+      for (int m = 0; m < MT; ++m) {
+        const int j = 16 * (wave * MT + m) + n16;
+        if (t < len && j < dv) a.y[((size_t)(first + t) * a.H + h) * dv + j] = acc[tb][m][r];
+      }
+    }
 }
 
 template <int NP, int DVP>
@@ -462,9 +488,13 @@ int launch_chunks(const SsdArgs<bf16_t>& a, int n_rows, int n_segs, const int32_
                   hipStream_t stream) {
   constexpr int PB = NP + 4, PV = DVP + 4;
   const size_t lds_local = ((size_t)kSeg * (PB + PV) + 2 * kSeg) * sizeof(float);
-  const size_t lds_read = ((size_t)kSeg * PV + 2 * kSeg) * sizeof(float);
+  const size_t lds_read = ((size_t)kSeg * (PV + kSeg + 4) + 2 * kSeg) * sizeof(float);
   if (lds_local > 48 * 1024) {
     hipError_t e = hipFuncSetAttribute((const void*)ssd_local_kernel<NP, DVP>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds_local);
+    if (e != hipSuccess) return tl_fail(TL_ERR_HIP, "ssd: %s", hipGetErrorString(e));
+  }
+  if (lds_read > 48 * 1024) {
+    hipError_t e = hipFuncSetAttribute((const void*)ssd_read_kernel<NP, DVP>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds_read);
     if (e != hipSuccess) return tl_fail(TL_ERR_HIP, "ssd: %s", hipGetErrorString(e));
   }
   const dim3 grid(n_segs, a.H);

@@ -117,6 +117,9 @@ class Engine:
                 "configuration; pass beyond_max_positions=True to run longer contexts all the same"
             )
         self.max_model_len = int(max_model_len or self.spec.max_positions)
+        learned = self.model.embedding.max_positions
+        if learned is not None and self.max_model_len > learned:
+            raise ValueError(f"max_model_len={self.max_model_len} exceeds the {learned} positions that the model has learned vectors for")
         self.page_size = page_size
         from ..kernels import ops
 

@@ -48,7 +48,7 @@ _CORE_SIGNATURES = {
     "tl_maps_join": [_P, _I, _P, _I, _I, _I, _F, _F, _F, _I, _P],
     "tl_expert_glu_rows": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
     "tl_expert_down_rows": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _P],
-    "tl_expert_gather": [_P, _P, _P, _I, _I, _I, _P, _P, _P, _P, _P, _I, _I, _P],
+    "tl_expert_gather": [_P, _P, _P, _I, _I, _I, _P, _P, _P, _I, _I, _P],
     "tl_pair_rows": [_P, _P, _P, _I, _I, _I, _I, _P],
     "tl_expert_combine": [_P, _I, _P, _P, _P, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _P],
     "tl_bias_gelu": [_P, _P, _I, _I, _I, _P],

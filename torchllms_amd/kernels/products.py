@@ -613,25 +613,34 @@ def pick(timed, use: str):
 
 def run_choice(choice, x: torch.Tensor, w: torch.Tensor, out_dtype: torch.dtype, leave_split: bool = False):
     if choice is None:
-        y = torch.nn.functional.linear(x, w)
-        return y if y.dtype == out_dtype else y.to(out_dtype)
+        if out_dtype != x.dtype:  # (32-bit results of bfloat16 inputs come from the product's own sums, never rounded on the way)
+            return torch.mm(x, w.t(), out_dtype=out_dtype)
+        return torch.nn.functional.linear(x, w)
     if choice[0] == "stream":
         return gemm_stream(x, w, out_dtype, choice[1])
     leave_split = leave_split and choice[2] > 1 and w.shape[0] % 4 == 0
     return gemm_wide(x, w, out_dtype, choice[1], choice[2], choice[3], leave_split)
 
 
-def linear(x: torch.Tensor, w: torch.Tensor, out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+def linear(x: torch.Tensor, w: torch.Tensor, out_dtype: Optional[torch.dtype] = None, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``x @ w.T``.  float32: the true 32-bit kernel.  bfloat16: for up to 128 rows (decode steps)
     one of the two MFMA kernels that are built around reading ``w`` once, or the BLAS library's
     matrix product, whichever was measured faster for the shape (``tune_linear``); for more rows the
     library, as the reference uses its library's (torchllms/models/networks.py:474-493).
-    ``out_dtype`` float32 asks for 32-bit results from bfloat16 inputs (logits)."""
+    ``out_dtype`` float32 asks for 32-bit results from bfloat16 inputs (logits).  ``out``: a row-major matrix of the
+    result's dtype that receives them (rows of a larger one will do)."""
     if x.dtype == torch.float32:
-        return gemm_f32(x, w)
-    _gpu(x, w)
+        return gemm_f32(x, w, out=out)
+    _gpu(x, w, out)
     out_dtype = out_dtype or x.dtype
-    return run_choice(linear_choice(x, w), x, w, out_dtype)
+    choice = linear_choice(x, w)
+    if out is None:
+        return run_choice(choice, x, w, out_dtype)
+    if out.shape != (x.shape[0], w.shape[0]) or out.dtype != out_dtype or out.stride(1) != 1:
+        raise KernelError(f"linear: out must be a row-major [{x.shape[0]}, {w.shape[0]}] matrix of {out_dtype}")
+    if choice is None:
+        return torch.mm(x, w.t(), out_dtype=out_dtype, out=out) if out_dtype != x.dtype else torch.mm(x, w.t(), out=out)
+    return out.copy_(run_choice(choice, x, w, out_dtype))
 
 
 def linear_to_sum(x: torch.Tensor, w: torch.Tensor, may_wait: bool = False):

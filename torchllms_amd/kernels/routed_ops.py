@@ -155,12 +155,10 @@ def expert_gather(x: torch.Tensor, ids: torch.Tensor, n_out: int, input_weights:
     top = ids.shape[1]
     if input_weights is not None:
         _input_weights(input_weights, n, top)
-    work = torch.zeros(3 * n_out + 1, dtype=torch.int32, device=x.device)
-    counts, offsets, cursor = work[:n_out], work[n_out : 2 * n_out + 1], work[2 * n_out + 1 :]
+    offsets = torch.empty(n_out + 1, dtype=torch.int32, device=x.device) if n else torch.zeros(n_out + 1, dtype=torch.int32, device=x.device)
     pos = torch.empty((n, top), dtype=torch.int32, device=x.device)
     rows = torch.empty((n * top, D), dtype=x.dtype, device=x.device)
-    check(core().tl_expert_gather(x.data_ptr(), ids.data_ptr(), _ptr(input_weights), n, top, n_out, counts.data_ptr(), offsets.data_ptr(), cursor.data_ptr(),
-                                  pos.data_ptr(), rows.data_ptr(), D, dtype_code(x.dtype), _stream()))
+    check(core().tl_expert_gather(x.data_ptr(), ids.data_ptr(), _ptr(input_weights), n, top, n_out, offsets.data_ptr(), pos.data_ptr(), rows.data_ptr(), D, dtype_code(x.dtype), _stream()))
     return rows, pos, offsets
 
 

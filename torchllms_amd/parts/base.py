@@ -278,6 +278,9 @@ class Registry(dict):
 
 
 class Embedding(Part):
+    #: how many positions it has rows for (None: positions do not enter it); no engine runs longer contexts
+    max_positions: Optional[int] = None
+
     def forward(self, tokens: torch.Tensor) -> torch.Tensor:
         """int32 token ids [n] -> [n, hidden]."""
         raise NotImplementedError

@@ -31,6 +31,7 @@ class TokenEmbedding(Embedding):
         self.scale = float(scale)
         self.stream_dtype = stream_dtype
         self.n_positions = int(positions)
+        self.max_positions = self.n_positions or None
         self.weight: Optional[torch.Tensor] = None
         self.positions: Optional[torch.Tensor] = None
 

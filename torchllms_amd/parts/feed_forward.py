@@ -226,11 +226,11 @@ class RoutedExperts(FeedForward):
             y = ops.expert_down_rows(ops.expert_glu_rows(rows, self.w_gu, offsets), self.w_down, offsets)
             return ops.expert_combine(y, pos, ids, weights, self.E, x, shared, gate)
         bounds = offsets.tolist()  # (the one place a step with prompts waits for the GPU)
-        parts = []
+        # (32-bit results: the weighted sum rounds once; the rows of experts that hand their input through lie behind all
+        # others and are never read)
+        y = torch.empty(rows.shape, dtype=torch.float32, device=rows.device)
         for e in range(self.E):
             lo, hi = bounds[e], bounds[e + 1]
             if hi > lo:
-                parts.append(ops.linear(ops.linear_glu(rows[lo:hi], self.w_gu[e]), self.w_down[e], out_dtype=torch.float32))
-        # (the rows of experts that hand their input through lie behind all others and are never read)
-        y = torch.cat(parts) if parts else rows  # (32-bit results: the weighted sum rounds once)
+                ops.linear(ops.linear_glu(rows[lo:hi], self.w_gu[e]), self.w_down[e], out_dtype=torch.float32, out=y[lo:hi])
         return ops.expert_combine(y, pos, ids, weights, self.E, x, shared, gate)
