@@ -674,9 +674,9 @@ def test_a_slot_that_is_used_again_starts_from_zero(tmp_path):
 
 @pytest.mark.parametrize("name", ["A", "B"])
 def test_long_decoding_from_recorded_steps(tmp_path, name):
-    """Three requests decode 150 tokens together, over window edges, through layers that use another's tensors: the steps are replayed from HIP
-    graphs after the first few, states move on with every replay, pages behind the windows go back, and the logits stay
-    the plain model's."""
+    """Three requests decode 150 tokens together, over window edges, through layers that use another's tensors: the steps
+    are replayed from HIP graphs after the first few, states move on with every replay, pages behind the windows go back,
+    and the logits stay the plain model's."""
     from torchllms_amd.engine import Engine, StepEntry
 
     requests = {f"d{i}": random_tokens(170 + 7 * i, models.CONFIGS[name]["vocab"], 60 + i) for i in range(3)}
